@@ -36,7 +36,11 @@
  *    version 7: hymeta_sink_attention_args ends with softcap / head_gate / head_gate_stride_t, hymeta_embed_rows_args with
  *    scale, hymeta_gated_rms_norm_args with groups / gate_act / gate_first, hymeta_moe_route_sigmoid_args with the grouped
  *    choice's fields; HYMETA_ROUTE_SOFTMAX_GROUPED; the parallel-layer, rotate-half, state-space and decayed-scan building
- *    blocks at the end of this file).
+ *    blocks at the end of this file;
+ *    version 8: hymeta_embed_rows_args ends with positions / pos_freqs / h_out, hymeta_norm_residual_args with h_out,
+ *    hymeta_sink_attention_args with elem_gate / elem_gate_stride_t, hymeta_activation_args with gate_rows /
+ *    gate_row_count; HYMETA_BIAS_LINEAR_DISTANCE, HYMETA_KV_SCALED_KEY, HYMETA_ACT_GELU_MUL / HYMETA_ACT_GELU_ROWS; the
+ *    scaled-key cache and the delta rule at the end of this file).
  *  - Every argument struct starts with `uint32_t struct_size`, which the caller
  *    sets to sizeof(the struct) of ITS declaration.  An entry point returns
  *    HYMETA_ERR_INVALID_ARG, before it reads any other field, when the value
@@ -54,7 +58,7 @@
 extern "C" {
 #endif
 
-#define HYMETA_ABI_VERSION 7
+#define HYMETA_ABI_VERSION 8
 
 typedef void* hymeta_stream_t;
 
@@ -1079,7 +1083,10 @@ int hymeta_p2p_destroy(hymeta_p2p_comm* comm);
  * neither read nor written).
  * ========================================================================================== */
 
-/* out[t] = table[token_ids[t]] (+ add), fp32 rows: the start of an fp32 residual stream. */
+/* out[t] = table[token_ids[t]] * scale (+ add), fp32 rows: the start of an fp32 residual stream.  With pos_freqs a
+ * sinusoidal vector of the row's position p is added besides: entry 2 i is sin(p pos_freqs[i]), entry 2 i + 1 its cosine
+ * (angles reduced in double precision, functions in fp32).  h_out: the rows once more, rounded to act_dtype (a first layer
+ * that reads the stream itself). */
 typedef struct hymeta_embed_rows_args {
   uint32_t struct_size;
   const int64_t* token_ids;    /* [num_tokens] */
@@ -1088,6 +1095,9 @@ typedef struct hymeta_embed_rows_args {
   float* out;                  /* [num_tokens, width] contiguous */
   int32_t num_tokens, width, vocab, act_dtype;
   float scale;                 /* the rows are multiplied by it (0: by 1) before add */
+  const int64_t* positions;    /* [num_tokens]; read with pos_freqs */
+  const double* pos_freqs;     /* [(width + 1) / 2] or NULL */
+  void* h_out;                 /* act_dtype [num_tokens, width] contiguous, or NULL */
 } hymeta_embed_rows_args;
 int hymeta_embed_rows(const hymeta_embed_rows_args* args, hymeta_stream_t stream);
 
@@ -1115,7 +1125,8 @@ typedef struct hymeta_norm_conv_args {
 int hymeta_norm_conv(const hymeta_norm_conv_args* args, hymeta_stream_t stream);
 
 /* x[t] += mult * y[t] / sqrt(mean(y[t]^2) + eps) * (weight_offset + weight) (+ post_add): a sublayer's
- * output through its output norm into the fp32 residual stream, in place. */
+ * output through its output norm into the fp32 residual stream, in place.  h_out: the new rows of x once more, rounded to
+ * act_dtype (the next sublayer's input where sublayers read the stream itself). */
 typedef struct hymeta_norm_residual_args {
   uint32_t struct_size;
   const void* y;               /* act_dtype [num_tokens, width], row stride y_stride_t */
@@ -1125,6 +1136,7 @@ typedef struct hymeta_norm_residual_args {
   int32_t num_tokens, width, act_dtype;
   float eps, weight_offset, mult;
   int64_t y_stride_t, x_stride_t;
+  void* h_out;                 /* act_dtype [num_tokens, width] contiguous, or NULL */
 } hymeta_norm_residual_args;
 int hymeta_norm_residual(const hymeta_norm_residual_args* args, hymeta_stream_t stream);
 
@@ -1171,7 +1183,8 @@ int hymeta_qk_norm_cache(const hymeta_qk_norm_cache_args* args, hymeta_stream_t 
 /* Causal attention of a step's queries over their sequences' paged keys (the step's own keys are in
  * the cache already), with a distance bias and an optional sink:
  *   s_ij = scale * q_i . k_j - bias(i - j),   j <= i   (and i - j <= window_left when window_left >= 0)
- *   bias_mode HYMETA_BIAS_NONE: 0;  HYMETA_BIAS_LOG_DISTANCE: bias_a[h] * ln(1 + bias_b[h] * (i - j))
+ *   bias_mode HYMETA_BIAS_NONE: 0;  HYMETA_BIAS_LOG_DISTANCE: bias_a[h] * ln(1 + bias_b[h] * (i - j));
+ *   HYMETA_BIAS_LINEAR_DISTANCE: bias_a[h] * (i - j)
  *   p_ij = exp(s_ij) / (sink + sum_j exp(s_ij)),  sink = exp(sink_logits[h]) (a key of that score, 0 without
  *   sink_logits, that has no value and is neither scaled nor biased) or 0
  *   out_i = sum_j p_ij v_j
@@ -1182,7 +1195,7 @@ int hymeta_qk_norm_cache(const hymeta_qk_norm_cache_args* args, hymeta_stream_t 
  * (hymeta_sink_attention_workspace_bytes) and merged by a second launch.
  * max_query_len / max_seq_len: upper bounds of the step's portion and sequence lengths (they size the
  * grids).  Everything else runs a wave per (row, head). */
-enum hymeta_bias_mode { HYMETA_BIAS_NONE = 0, HYMETA_BIAS_LOG_DISTANCE = 1 };
+enum hymeta_bias_mode { HYMETA_BIAS_NONE = 0, HYMETA_BIAS_LOG_DISTANCE = 1, HYMETA_BIAS_LINEAR_DISTANCE = 2 };
 /* What a key/value head's part of a cache row holds.  KEY_THEN_VALUE: head_dim key elements followed by v_dim value
  * elements (hymeta_qk_norm_cache).  VALUE_IN_KEY: head_dim elements, of which the first v_dim are also the value (a
  * latent shared by keys and values followed by a rotated key part: hymeta_latent_kv_prep); v_dim <= head_dim.  With
@@ -1193,8 +1206,13 @@ enum hymeta_bias_mode { HYMETA_BIAS_NONE = 0, HYMETA_BIAS_LOG_DISTANCE = 1 };
  * v_dim elements; query head h reads value h / (num_heads / num_kv_heads) (hymeta_talk_qkv_prep: queries that were
  * mixed across heads against the concatenated keys of the key/value heads).  bf16 rows with head_dim 128 / 256 / 512 and
  * v_dim 64 / 128 run on the matrix cores.
+ * SCALED_KEY: per key/value head ONE vector of head_dim = v_dim elements that is the value, and also the key up to a factor
+ * per (row, head) that multiplies q . k (a normed key whose value is the unnormed one: hymeta_scaled_key_cache); a row is
+ * num_kv_heads such vectors, then from the next multiple of 4 bytes on num_kv_heads fp32 factors, padded to a multiple of
+ * 16 bytes.  bf16 rows with head_dim 32 / 64 / 96 / 128, no or a linear bias and no cap run on the matrix cores.
  * keep_first (with window_left >= 0): keys j < keep_first stay visible to every later query, at their own positions. */
-enum hymeta_kv_layout { HYMETA_KV_KEY_THEN_VALUE = 0, HYMETA_KV_VALUE_IN_KEY = 1, HYMETA_KV_SHARED_KEY = 2 };
+enum hymeta_kv_layout { HYMETA_KV_KEY_THEN_VALUE = 0, HYMETA_KV_VALUE_IN_KEY = 1, HYMETA_KV_SHARED_KEY = 2,
+                        HYMETA_KV_SCALED_KEY = 3 };
 typedef struct hymeta_sink_attention_args {
   uint32_t struct_size;
   const void* q;               /* act_dtype [num_tokens, num_heads, head_dim], strides q_stride_t / head_dim */
@@ -1204,7 +1222,7 @@ typedef struct hymeta_sink_attention_args {
   const int32_t* query_start_loc;  /* [num_seqs + 1] */
   const int32_t* seq_lens;         /* [num_seqs]: keys of the sequence, this step's rows included */
   const float* bias_a;         /* [num_heads] */
-  const float* bias_b;         /* [num_heads] */
+  const float* bias_b;         /* [num_heads] (HYMETA_BIAS_LOG_DISTANCE) */
   void* workspace;
   size_t workspace_bytes;
   int32_t num_tokens, num_seqs, num_heads, num_kv_heads, head_dim, v_dim, block_size, act_dtype;
@@ -1218,6 +1236,9 @@ typedef struct hymeta_sink_attention_args {
   const void* head_gate;       /* act_dtype [num_tokens, num_heads], row stride head_gate_stride_t, or NULL: head h's
                                   output of row t is multiplied by sigmoid(head_gate[t, h]) */
   int64_t head_gate_stride_t;
+  const void* elem_gate;       /* act_dtype [num_tokens, num_heads * v_dim], row stride elem_gate_stride_t, or NULL: the
+                                  output is multiplied element by element by sigmoid(elem_gate) */
+  int64_t elem_gate_stride_t;
 } hymeta_sink_attention_args;
 size_t hymeta_sink_attention_workspace_bytes(int32_t num_seqs, int32_t num_heads, int32_t num_kv_heads, int32_t v_dim,
                                              int32_t max_seq_len);
@@ -1406,9 +1427,12 @@ int hymeta_gated_rms_norm(const hymeta_gated_rms_norm_args* args, hymeta_stream_
  *   HYMETA_ACT_SIGMOID_MUL  x [rows, n], gate [rows, n]: out = x * sigmoid(gate)
  *   HYMETA_ACT_SILU_MUL     x [rows, 2 n] (gate columns, then up columns): out = gate sigmoid(gate) up
  *   HYMETA_ACT_RELU2        x [rows, n]: out = max(x, 0)^2
+ *   HYMETA_ACT_GELU_MUL     x [rows, 2 n] (gate columns, then up columns): out = gelu(gate) up, gelu in its tanh form:
+ *                           gelu(z) = z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))
+ *   HYMETA_ACT_GELU_ROWS    x [rows, n], gate [gate_row_count, >= n] (a table): out = gelu(x) * gate[gate_rows[row]]
  * num_rows_dev: optional device count of the rows in use; NULL: num_rows. */
 enum hymeta_act_kind { HYMETA_ACT_CLAMPED_GLU = 0, HYMETA_ACT_XIELU = 1, HYMETA_ACT_SIGMOID_MUL = 2, HYMETA_ACT_SILU_MUL = 3,
-                       HYMETA_ACT_RELU2 = 4 };
+                       HYMETA_ACT_RELU2 = 4, HYMETA_ACT_GELU_MUL = 5, HYMETA_ACT_GELU_ROWS = 6 };
 typedef struct hymeta_activation_args {
   uint32_t struct_size;
   const void* x;               /* [rows, n or 2 n], row stride x_stride */
@@ -1418,6 +1442,8 @@ typedef struct hymeta_activation_args {
   int32_t kind, num_rows, n, act_dtype;
   float p0, p1;                /* CLAMPED_GLU: limit, alpha;  XIELU: a_pos, a_neg */
   int64_t x_stride, gate_stride, out_stride;
+  const int64_t* gate_rows;    /* HYMETA_ACT_GELU_ROWS: [rows], row of `gate` per row of x (clamped into the table) */
+  int64_t gate_row_count;
 } hymeta_activation_args;
 int hymeta_activation(const hymeta_activation_args* args, hymeta_stream_t stream);
 
@@ -1641,6 +1667,68 @@ typedef struct hymeta_decay_scan_args {
 /* > 0 for steps with long portions: they run in segments side by side (summarise / chain / apply: three launches). */
 size_t hymeta_decay_scan_workspace_bytes(int32_t num_seqs, int32_t num_heads, int32_t head_dim, int32_t v_dim, int32_t max_query_len);
 int hymeta_decay_scan(const hymeta_decay_scan_args* args, hymeta_stream_t stream);
+
+/* ------------------------------------------------------------------------
+ * Building blocks of designs that norm what a sublayer adds (and not what it reads), with attention whose values are its
+ * unnormed keys, and gated delta-rule layers.
+ * ---------------------------------------------------------------------- */
+
+/* Between a fused q | k (| ...) projection and HYMETA_KV_SCALED_KEY attention, per token, one launch:
+ *   q[t, h] <- q[t, h] / sqrt(mean(q[t, h]^2) + eps) * q_weight * k_weight * temperature(positions[t])      (in place)
+ *   cache row at slot_mapping[t] <- the keys as they are, and 1 / sqrt(mean(k[t, g]^2) + eps) per key/value head
+ * so that q . k times the stored factor is the product of the normed query and the normed key (both norms with their own
+ * per-column weight).  temperature(p) = 1 + temp_coef ln(floor((p + 1) / temp_every) + 1); temp_coef 0: 1.
+ * slot_mapping[t] < 0 or NULL: nothing is stored. */
+typedef struct hymeta_scaled_key_cache_args {
+  uint32_t struct_size;
+  void* qk;                    /* act_dtype [num_tokens, H D + G D (+ more)], row stride qk_stride_t */
+  const float* q_weight;       /* [head_dim] */
+  const float* k_weight;       /* [head_dim] */
+  void* kv_cache;              /* act_dtype [num_blocks, block_size, row elements] (enum hymeta_kv_layout), 16-byte aligned */
+  const int64_t* slot_mapping; /* [num_tokens] or NULL */
+  const int64_t* positions;    /* [num_tokens]; read when temp_coef != 0 */
+  double temp_every;
+  int32_t num_tokens, num_heads, num_kv_heads, head_dim, block_size, act_dtype;
+  float eps, temp_coef;
+  int64_t num_blocks, qk_stride_t;
+} hymeta_scaled_key_cache_args;
+int hymeta_scaled_key_cache(const hymeta_scaled_key_cache_args* args, hymeta_stream_t stream);
+
+/* Gated delta rule over a step's rows, the state fp32 [slots, H, D, Dv] carried per sequence.  With unit vectors
+ * k' = k / sqrt(sum(k^2) + unit_eps), q' = q_scale q / sqrt(sum(q^2) + unit_eps), beta = sigmoid(beta_logit[t, h]) and
+ * a = exp2(log2_decay[t, h]), in this order:
+ *   S <- a S;   u = beta (v - S^T k');   S <- S + k' u^T;   o = S^T q'
+ * query / key head of head h: h / (num_heads / num_qk_heads).  Without norm_weight: out fp32 = o.  With it (every sequence
+ * of the step brings one row, max_query_len == 1, v_dim in whole fours that divide 256 fours):
+ *   out act_dtype = o / sqrt(mean(o^2) + norm_eps) * norm_weight * silu(gate[t, h])
+ * Sequences with one row run a step kernel; bf16 portions of 8 rows and more run HYMETA_DELTA_CHUNK rows at a time on the
+ * matrix cores where head_dim is 32 / 64 / 96 / 128 and v_dim in whole 32s (a launch over all chunks that solves each
+ * chunk's triangular system, then one that carries the state through them, products of fp32 quantities in hi + lo bf16
+ * parts); everything else token by token. */
+#define HYMETA_DELTA_CHUNK 64
+typedef struct hymeta_delta_rule_args {
+  uint32_t struct_size;
+  const void* q;               /* act_dtype [num_tokens, num_qk_heads, head_dim], row stride q_stride_t */
+  const void* k;               /* likewise, row stride k_stride_t */
+  const void* v;               /* act_dtype [num_tokens, num_heads, v_dim], row stride v_stride_t */
+  const void* beta_logit;      /* act_dtype [num_tokens, num_heads], row stride beta_stride_t */
+  const float* log2_decay;     /* [num_tokens, num_heads] contiguous */
+  float* state;
+  void* out;                   /* fp32 (norm_weight: act_dtype) [num_tokens, num_heads * v_dim] contiguous */
+  const float* norm_weight;    /* [v_dim] or NULL */
+  const void* gate;            /* act_dtype [num_tokens, num_heads * v_dim], row stride gate_stride_t (norm_weight) */
+  const int32_t* query_start_loc;
+  const int32_t* context_lens;
+  const int32_t* slot_idx;
+  int32_t num_tokens, num_seqs, num_heads, num_qk_heads, head_dim, v_dim, act_dtype, max_query_len;
+  float q_scale, unit_eps, norm_eps;
+  int64_t q_stride_t, k_stride_t, v_stride_t, beta_stride_t, gate_stride_t;
+  void* workspace;             /* hymeta_delta_rule_workspace_bytes(...) bytes, or NULL when that is 0 */
+  size_t workspace_bytes;
+} hymeta_delta_rule_args;
+size_t hymeta_delta_rule_workspace_bytes(int32_t num_tokens, int32_t num_seqs, int32_t num_heads, int32_t num_qk_heads, int32_t head_dim,
+                                         int32_t v_dim, int32_t act_dtype, int32_t max_query_len);
+int hymeta_delta_rule(const hymeta_delta_rule_args* args, hymeta_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -15,15 +15,40 @@ constexpr int kNormThreads = 256;
 constexpr int kNormWaves = kNormThreads / 64;
 constexpr int kMaxPerThread = 32;          // width <= 256 * 32 channels
 
+// Sine and cosine of pos * freq: the angle in double precision, brought into [-pi, pi]; the functions are the fp32 ones on
+// the remainder.
+__device__ __forceinline__ void position_pair(int64_t pos, double freq, float& sine, float& cosine) {
+  constexpr double kTwoPi = 6.283185307179586476925286766559, kInvTwoPi = 0.15915494309189533576888376337251;
+  const double ang = static_cast<double>(pos) * freq;
+  const float r = static_cast<float>(fma(-kTwoPi, rint(ang * kInvTwoPi), ang));
+  sine = sinf(r);
+  cosine = cosf(r);
+}
+
+// A thread takes pairs of columns (2 i, 2 i + 1): one angle each.
 template <typename A>
 __global__ __launch_bounds__(kNormThreads) void embed_rows_kernel(hymeta_embed_rows_args a) {
+  typedef typename A::elem elem;
   const int t = blockIdx.x;
   int64_t tok = a.token_ids[t];
   if (tok < 0 || tok >= a.vocab) tok = 0;          // ids are validated on the host; never read out of the table
-  const typename A::elem* row = static_cast<const typename A::elem*>(a.table) + tok * a.width;
+  const elem* row = static_cast<const elem*>(a.table) + tok * a.width;
   float* out = a.out + static_cast<int64_t>(t) * a.width;
+  elem* h = a.h_out ? static_cast<elem*>(a.h_out) + static_cast<int64_t>(t) * a.width : nullptr;
   const float scale = a.scale != 0.f ? a.scale : 1.f;
-  for (int c = threadIdx.x; c < a.width; c += kNormThreads) out[c] = A::ld(row + c) * scale + (a.add ? a.add[c] : 0.f);
+  const int64_t pos = a.pos_freqs ? a.positions[t] : 0;
+  for (int i = threadIdx.x; 2 * i < a.width; i += kNormThreads) {
+    float wave[2] = {0.f, 0.f};
+    if (a.pos_freqs) position_pair(pos, a.pos_freqs[i], wave[0], wave[1]);
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+      const int c = 2 * i + e;
+      if (c >= a.width) continue;
+      const float v = A::ld(row + c) * scale + (a.add ? a.add[c] : 0.f) + wave[e];
+      out[c] = v;
+      if (h) A::st(h + c, v);
+    }
+  }
 }
 
 __device__ __forceinline__ int seq_of_row_fast(const hymeta_norm_conv_args& a, int t);
@@ -282,13 +307,52 @@ __global__ __launch_bounds__(kNormThreads) void norm_conv_kernel(hymeta_norm_con
   }
 }
 
-template <typename A>
+// Fours: a thread takes runs of four consecutive columns (rows of up to 4 * kNormThreads * kResidualRuns columns, pointers
+// and strides in whole fours), whose loads of y, x and the weight are in flight together.
+constexpr int kResidualRuns = 4;
+
+template <typename A, bool Fours>
 __global__ __launch_bounds__(kNormThreads) void norm_residual_kernel(hymeta_norm_residual_args a) {
   typedef typename A::elem elem;
   __shared__ float red[kNormWaves];
   const int64_t t = blockIdx.x;
   const elem* y = static_cast<const elem*>(a.y) + t * a.y_stride_t;
   float* x = a.x + t * a.x_stride_t;
+  elem* h = a.h_out ? static_cast<elem*>(a.h_out) + t * a.width : nullptr;
+  if constexpr (Fours) {
+    float v[kResidualRuns][4], xv[kResidualRuns][4];
+    float ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < kResidualRuns; ++u) {
+      const int c = 4 * (threadIdx.x + u * kNormThreads);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[u][e] = 0.f, xv[u][e] = 0.f;
+      if (c < a.width) A::ld4(y + c, v[u]), ActF32::ld4(x + c, xv[u]);
+    }
+#pragma unroll
+    for (int u = 0; u < kResidualRuns; ++u)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss = fmaf(v[u][e], v[u][e], ss);
+    ss = block_sum<kNormWaves>(ss, red);
+    const float inv = 1.f / sqrtf(ss / static_cast<float>(a.width) + a.eps);
+#pragma unroll
+    for (int u = 0; u < kResidualRuns; ++u) {
+      const int c = 4 * (threadIdx.x + u * kNormThreads);
+      if (c >= a.width) continue;
+      float w[4], add[4] = {0.f, 0.f, 0.f, 0.f};
+      ActF32::ld4(a.weight + c, w);
+      if (a.post_add) ActF32::ld4(a.post_add + c, add);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        float r = xv[u][e] + a.mult * (v[u][e] * inv * (a.weight_offset + w[e]));
+        if (a.post_add) r += add[e];
+        xv[u][e] = r;
+      }
+      ActF32::st4(x + c, xv[u]);
+      if (h) A::st4(h + c, xv[u]);
+    }
+    return;
+  }
   float v[kMaxPerThread];
   float ss = 0.f;
 #pragma unroll
@@ -306,6 +370,7 @@ __global__ __launch_bounds__(kNormThreads) void norm_residual_kernel(hymeta_norm
       float r = x[c] + a.mult * (v[u] * inv * (a.weight_offset + a.weight[c]));
       if (a.post_add) r += a.post_add[c];
       x[c] = r;
+      if (h) A::st(h + c, r);
     }
   }
 }
@@ -322,7 +387,7 @@ extern "C" int hymeta_embed_rows(const hymeta_embed_rows_args* args, hymeta_stre
   if (a.num_tokens < 0 || a.width <= 0 || a.vocab <= 0) return HYMETA_ERR_INVALID_ARG;
   if (!act_dtype_ok(a.act_dtype)) return HYMETA_ERR_UNSUPPORTED;
   if (a.num_tokens == 0) return HYMETA_OK;
-  if (!a.token_ids || !a.table || !a.out) return HYMETA_ERR_INVALID_ARG;
+  if (!a.token_ids || !a.table || !a.out || (a.pos_freqs && !a.positions)) return HYMETA_ERR_INVALID_ARG;
   hipStream_t st = begin_launches(stream);
   if (a.act_dtype == HYMETA_BF16) hipLaunchKernelGGL(embed_rows_kernel<ActBf16>, dim3(a.num_tokens), dim3(kNormThreads), 0, st, a);
   else hipLaunchKernelGGL(embed_rows_kernel<ActF32>, dim3(a.num_tokens), dim3(kNormThreads), 0, st, a);
@@ -363,7 +428,17 @@ extern "C" int hymeta_norm_residual(const hymeta_norm_residual_args* args, hymet
   if (a.num_tokens == 0) return HYMETA_OK;
   if (!a.y || !a.weight || !a.x || a.x_stride_t < a.width || a.y_stride_t < a.width) return HYMETA_ERR_INVALID_ARG;
   hipStream_t st = begin_launches(stream);
-  if (a.act_dtype == HYMETA_BF16) hipLaunchKernelGGL(norm_residual_kernel<ActBf16>, dim3(a.num_tokens), dim3(kNormThreads), 0, st, a);
-  else hipLaunchKernelGGL(norm_residual_kernel<ActF32>, dim3(a.num_tokens), dim3(kNormThreads), 0, st, a);
+  const int bytes = a.act_dtype == HYMETA_BF16 ? 2 : 4;
+  auto fours = [](const void* p, int64_t stride, int eb) { return p == nullptr || (reinterpret_cast<uintptr_t>(p) % (4 * eb) == 0 && stride % 4 == 0); };
+  const bool vec = a.width % 4 == 0 && a.width <= 4 * kNormThreads * kResidualRuns && fours(a.y, a.y_stride_t, bytes) && fours(a.x, a.x_stride_t, 4) &&
+                   fours(a.weight, 0, 4) && fours(a.post_add, 0, 4) && fours(a.h_out, 0, bytes);
+  const dim3 grid(a.num_tokens), block(kNormThreads);
+  if (a.act_dtype == HYMETA_BF16) {
+    if (vec) hipLaunchKernelGGL((norm_residual_kernel<ActBf16, true>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((norm_residual_kernel<ActBf16, false>), grid, block, 0, st, a);
+  } else {
+    if (vec) hipLaunchKernelGGL((norm_residual_kernel<ActF32, true>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((norm_residual_kernel<ActF32, false>), grid, block, 0, st, a);
+  }
   return launch_status();
 }

@@ -4,6 +4,10 @@
 // Scores, the running maximum, the weights and the weighted sum of the values are fp32 whatever the
 // activation type.  The sink is a key of score 0 without a value: the running maximum starts at 0
 // and the denominator at exp(0 - 0) = 1, everything else is the ordinary streaming softmax.
+//
+// Rows of HYMETA_KV_SCALED_KEY hold ONE vector per key/value head that is both: the projected key, which is the value,
+// and its inverse root mean square, by which the score of the normed key differs from the score of the stored one (the
+// norm's weight rides in the queries).  A page then holds half of what keys and values apart would take.
 #include "act_types.h"
 
 namespace hymeta {
@@ -56,7 +60,81 @@ __global__ __launch_bounds__(256) void qk_norm_cache_kernel(hymeta_qk_norm_cache
   }
 }
 
+// A row of HYMETA_KV_SCALED_KEY: num_kv_heads keys of head_dim elements, then (from the next multiple of 4 bytes on) an
+// fp32 scale per key/value head, the whole padded to 16 bytes.
+struct ScaledRow {
+  int64_t elems;          // elements of the activation type per row
+  int64_t scale_bytes;    // where the scales start, in bytes
+};
+__host__ __device__ inline ScaledRow scaled_row(int num_kv_heads, int head_dim, int elem_bytes) {
+  const int64_t at = (static_cast<int64_t>(num_kv_heads) * head_dim * elem_bytes + 3) / 4 * 4;
+  return ScaledRow{(at + 4 * static_cast<int64_t>(num_kv_heads) + 15) / 16 * 16 / elem_bytes, at};
+}
+
+// grid = tokens.  `Lanes` neighbouring lanes (a power of two) share a head, four elements each (Vec), or the lanes of a wave
+// stride over it: query heads (normed, times q_weight, k_weight and the temperature of the row's position, in place), then
+// key heads (stored as they are, with their inverse root mean square).
+template <typename A, bool Vec>
+__global__ __launch_bounds__(256) void scaled_key_cache_kernel(hymeta_scaled_key_cache_args a, int lanes) {
+  typedef typename A::elem elem;
+  const int64_t t = blockIdx.x;
+  const int H = a.num_heads, G = a.num_kv_heads, D = a.head_dim;
+  const int sub = threadIdx.x & (lanes - 1), first = threadIdx.x / lanes, step = 256 / lanes;
+  elem* row = static_cast<elem*>(a.qk) + t * a.qk_stride_t;
+  const int64_t slot = a.slot_mapping ? a.slot_mapping[t] : -1;
+  const bool store = slot >= 0 && slot < a.num_blocks * a.block_size;
+  const ScaledRow lay = scaled_row(G, D, sizeof(elem));
+  elem* cache = store ? static_cast<elem*>(a.kv_cache) + slot * lay.elems : nullptr;
+  float temp = 1.f;
+  if (a.temp_coef != 0.f) {
+    // floor of the exact quotient: a double holds positions and periods exactly, and no quotient of two of them rounds up
+    // to the next integer
+    const double n = floor((static_cast<double>(a.positions[t]) + 1.0) / a.temp_every) + 1.0;
+    temp = 1.f + a.temp_coef * logf(static_cast<float>(n));
+  }
+  for (int task = first; task < H + G; task += step) {
+    const bool is_q = task < H;
+    elem* src = row + static_cast<int64_t>(task) * D;
+    float ss = 0.f, v[4];
+    if (Vec) {
+      const bool on = 4 * sub < D;
+      if (on) A::ld4(src + 4 * sub, v);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss = on ? fmaf(v[e], v[e], ss) : ss;
+    } else {
+      for (int d = sub; d < D; d += lanes) {
+        const float x = A::ld(src + d);
+        ss = fmaf(x, x, ss);
+      }
+    }
+    for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float inv = 1.f / sqrtf(ss / static_cast<float>(D) + a.eps);
+    if (is_q) {
+      const float f = inv * temp;
+      if (Vec) {
+        if (4 * sub < D) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] *= f * a.q_weight[4 * sub + e] * a.k_weight[4 * sub + e];
+          A::st4(src + 4 * sub, v);
+        }
+      } else {
+        for (int d = sub; d < D; d += lanes) A::st(src + d, A::ld(src + d) * f * a.q_weight[d] * a.k_weight[d]);
+      }
+    } else if (store) {
+      const int g = task - H;
+      elem* dst = cache + static_cast<int64_t>(g) * D;
+      if (Vec) {
+        if (4 * sub < D) A::st4(dst + 4 * sub, v);
+      } else {
+        for (int d = sub; d < D; d += lanes) dst[d] = src[d];
+      }
+      if (sub == 0) reinterpret_cast<float*>(reinterpret_cast<char*>(cache) + lay.scale_bytes)[g] = inv;
+    }
+  }
+}
+
 __device__ __forceinline__ float distance_bias(int mode, float a, float b, int dist) {
+  if (mode == HYMETA_BIAS_LINEAR_DISTANCE) return a * static_cast<float>(dist);
   return mode == HYMETA_BIAS_LOG_DISTANCE ? a * log1pf(b * static_cast<float>(dist)) : 0.f;
 }
 
@@ -82,10 +160,13 @@ __global__ __launch_bounds__(64) void sink_attention_rows_kernel(hymeta_sink_att
   // where the head's key and value lie in a cache row: a key followed by its value per key/value head; a key whose first Dv
   // elements are the value; or one key for all heads followed by the key/value heads' values
   int64_t row_elems, key_off, val_off;
-  if (a.kv_layout == HYMETA_KV_SHARED_KEY) row_elems = D + static_cast<int64_t>(G) * Dv, key_off = 0, val_off = D + static_cast<int64_t>(g) * Dv;
+  const bool scaled = a.kv_layout == HYMETA_KV_SCALED_KEY;
+  const ScaledRow lay = scaled_row(G, D, sizeof(elem));
+  if (scaled) row_elems = lay.elems, key_off = static_cast<int64_t>(g) * D, val_off = key_off;
+  else if (a.kv_layout == HYMETA_KV_SHARED_KEY) row_elems = D + static_cast<int64_t>(G) * Dv, key_off = 0, val_off = D + static_cast<int64_t>(g) * Dv;
   else if (a.kv_layout == HYMETA_KV_VALUE_IN_KEY) row_elems = static_cast<int64_t>(G) * D, key_off = static_cast<int64_t>(g) * D, val_off = key_off;
   else row_elems = static_cast<int64_t>(G) * (D + Dv), key_off = static_cast<int64_t>(g) * (D + Dv), val_off = key_off + D;
-  const float ba = a.bias_mode ? a.bias_a[h] : 0.f, bb = a.bias_mode ? a.bias_b[h] : 0.f;
+  const float ba = a.bias_mode ? a.bias_a[h] : 0.f, bb = a.bias_mode == HYMETA_BIAS_LOG_DISTANCE ? a.bias_b[h] : 0.f;
   // the sink: a key of score sink_logits[h] (0 without) that has no value
   float m = a.sink ? (a.sink_logits ? a.sink_logits[h] : 0.f) : -INFINITY, l = a.sink ? 1.f : 0.f;
   float acc[kMaxVChunks] = {};
@@ -106,6 +187,7 @@ __global__ __launch_bounds__(64) void sink_attention_rows_kernel(hymeta_sink_att
         const elem* k = cache + roff + key_off;
         float dot = 0.f;
         for (int d = 0; d < D; ++d) dot = fmaf(s_q[d], A::ld(k + d), dot);
+        if (scaled) dot *= reinterpret_cast<const float*>(reinterpret_cast<const char*>(cache + roff) + lay.scale_bytes)[g];
         sc = dot * a.scale;
         if (a.softcap > 0.f) sc = a.softcap * tanhf(sc / a.softcap);
         sc -= distance_bias(a.bias_mode, ba, bb, pos - j);
@@ -138,7 +220,11 @@ __global__ __launch_bounds__(64) void sink_attention_rows_kernel(hymeta_sink_att
 #pragma unroll
   for (int cc = 0; cc < kMaxVChunks; ++cc) {
     const int c = cc * 64 + lane;
-    if (cc < nvc && c < Dv) A::st(out + c, acc[cc] * inv);
+    if (cc < nvc && c < Dv) {
+      float v = acc[cc] * inv;
+      if (a.elem_gate) v *= sigmoid_exact(A::ld(static_cast<const elem*>(a.elem_gate) + static_cast<int64_t>(t) * a.elem_gate_stride_t + static_cast<int64_t>(h) * Dv + c));
+      A::st(out + c, v);
+    }
   }
 }
 
@@ -197,17 +283,22 @@ struct MfmaSmem {
 // of threads that hold the same keys over the banks; the reader applies the same permutation.
 // Layout (enum hymeta_kv_layout).  VALUE_IN_KEY: a head's part of a cache row is its key alone (D elements), whose first DV
 // elements are also its value.  SHARED_KEY: a row is one key of D elements for all heads, then num_kv_heads values of DV.
+// SCALED_KEY: a head's part is one vector that is key and value (D == DV), read from memory once and stored into both images,
+// and the keys' scales go into an array of their own.
 template <int D, int DV, int Threads, int Layout>
 struct TileStage {
   static constexpr bool VinK = Layout == HYMETA_KV_VALUE_IN_KEY, Shared = Layout == HYMETA_KV_SHARED_KEY;
+  static constexpr bool Scaled = Layout == HYMETA_KV_SCALED_KEY;
   static constexpr int kKeyChunksPerRow = D / 8, kValChunksPerRow = DV / 8;
   static constexpr int kKeyChunks = kTileKeys * kKeyChunksPerRow;
   static constexpr int kKeyPerThread = (kKeyChunks + Threads - 1) / Threads;
   static constexpr int kValBlocks = (kTileKeys / 4) * kValChunksPerRow;       // (4 keys) x (8 channels) each
-  static constexpr int kHeadElems = VinK ? D : D + DV, kValueAt = VinK ? 0 : D;
-  static_assert(D % 32 == 0 && DV % 16 == 0 && kValBlocks <= Threads && (!VinK || DV <= D), "the staging roles fit the workgroup");
-  u32x4 rk[kKeyPerThread];
+  static constexpr int kHeadElems = (VinK || Scaled) ? D : D + DV, kValueAt = (VinK || Scaled) ? 0 : D;
+  static_assert(D % 32 == 0 && DV % 16 == 0 && kValBlocks <= Threads && (!VinK || DV <= D) && (!Scaled || DV == D) && kTileKeys <= Threads,
+                "the staging roles fit the workgroup");
+  u32x4 rk[Scaled ? 1 : kKeyPerThread];
   u32x4 rv[4];
+  float rs = 0.f;               // (SCALED_KEY) the scale of key j0 + threadIdx.x
   int value_at = kValueAt;      // where the staged value columns start in a head's part of a row
 
   // Pages hold a power of two of rows here (the host sends other sizes to the plain kernel).  A page of 64 rows or more
@@ -226,7 +317,7 @@ struct TileStage {
     Pages p;
     p.cache = static_cast<const uint16_t*>(a.kv_cache);
     p.bt = bt;
-    p.row_elems = Shared ? D + static_cast<int64_t>(a.num_kv_heads) * DV : static_cast<int64_t>(a.num_kv_heads) * kHeadElems;
+    p.row_elems = Scaled ? scaled_row(a.num_kv_heads, D, 2).elems : Shared ? D + static_cast<int64_t>(a.num_kv_heads) * DV : static_cast<int64_t>(a.num_kv_heads) * kHeadElems;
     p.head_off = Shared ? 0 : static_cast<int64_t>(g) * kHeadElems;
     p.shift = __builtin_ctz(a.block_size);
     p.mask = a.block_size - 1;
@@ -243,12 +334,19 @@ struct TileStage {
 
   __device__ __forceinline__ void issue(const hymeta_sink_attention_args& a, const int32_t* bt, int g, int j0, int last) {
     const Pages p = pages(a, bt, g, j0);
+    if constexpr (Scaled) {
+      const int j = j0 + static_cast<int>(threadIdx.x);
+      rs = 0.f;
+      if (static_cast<int>(threadIdx.x) < kTileKeys && j <= last)
+        rs = reinterpret_cast<const float*>(reinterpret_cast<const char*>(row_ptr(p, j0, j) - p.head_off) + scaled_row(a.num_kv_heads, D, 2).scale_bytes)[g];
+    } else {
 #pragma unroll
-    for (int i = 0; i < kKeyPerThread; ++i) {
-      const int idx = i * Threads + threadIdx.x;
-      const int j = j0 + idx / kKeyChunksPerRow;
-      rk[i] = u32x4{0u, 0u, 0u, 0u};
-      if (j <= last && (kKeyChunks % Threads == 0 || idx < kKeyChunks)) rk[i] = ld16g(row_ptr(p, j0, j) + (idx % kKeyChunksPerRow) * 8);
+      for (int i = 0; i < kKeyPerThread; ++i) {
+        const int idx = i * Threads + threadIdx.x;
+        const int j = j0 + idx / kKeyChunksPerRow;
+        rk[i] = u32x4{0u, 0u, 0u, 0u};
+        if (j <= last && (kKeyChunks % Threads == 0 || idx < kKeyChunks)) rk[i] = ld16g(row_ptr(p, j0, j) + (idx % kKeyChunksPerRow) * 8);
+      }
     }
     if (static_cast<int>(threadIdx.x) < kValBlocks) {
       const int ch = threadIdx.x % kValChunksPerRow, grp = threadIdx.x / kValChunksPerRow;
@@ -261,12 +359,21 @@ struct TileStage {
     }
   }
 
-  __device__ __forceinline__ void commit(MfmaSmem<D, DV>& sm) const {
+  __device__ __forceinline__ void commit(MfmaSmem<D, DV>& sm, float* scales) const {
+    if constexpr (Scaled) {
+      if (static_cast<int>(threadIdx.x) < kTileKeys) scales[threadIdx.x] = rs;
+      if (static_cast<int>(threadIdx.x) < kValBlocks) {
+        const int ch = threadIdx.x % kValChunksPerRow, grp = threadIdx.x / kValChunksPerRow;
 #pragma unroll
-    for (int i = 0; i < kKeyPerThread; ++i) {
-      const int idx = i * Threads + threadIdx.x;
-      if (kKeyChunks % Threads == 0 || idx < kKeyChunks)
-        st16(&sm.k[(idx / kKeyChunksPerRow) * MfmaSmem<D, DV>::kPitchK + (idx % kKeyChunksPerRow) * 8], rk[i]);
+        for (int i = 0; i < 4; ++i) st16(&sm.k[(4 * grp + i) * MfmaSmem<D, DV>::kPitchK + ch * 8], rv[i]);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < kKeyPerThread; ++i) {
+        const int idx = i * Threads + threadIdx.x;
+        if (kKeyChunks % Threads == 0 || idx < kKeyChunks)
+          st16(&sm.k[(idx / kKeyChunksPerRow) * MfmaSmem<D, DV>::kPitchK + (idx % kKeyChunksPerRow) * 8], rk[i]);
+      }
     }
     if (static_cast<int>(threadIdx.x) < kValBlocks) {
       const int ch = threadIdx.x % kValChunksPerRow, grp = threadIdx.x / kValChunksPerRow;
@@ -313,9 +420,11 @@ __device__ __forceinline__ float tanh_fast(float x) {
   return 1.f - 2.f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x * 2.8853900817779268f) + 1.f);
 }
 
-template <int D, int DV, int RB, int NKS, bool Masked>
-__device__ __forceinline__ void attend_tile(WaveRows<D, DV, RB>& w, const MfmaSmem<D, DV>& sm, const hymeta_sink_attention_args& a,
-                                            int j0, int ks_lo) {
+// Scaled (SCALED_KEY rows): `scales` holds a factor per key of the tile, the bias is linear in the distance (its
+// coefficient, in the base-2 domain, in w.ba) and there is no cap.
+template <int D, int DV, int RB, int NKS, bool Masked, bool Scaled>
+__device__ __forceinline__ void attend_tile(WaveRows<D, DV, RB>& w, const MfmaSmem<D, DV>& sm, const float* scales,
+                                            const hymeta_sink_attention_args& a, int j0, int ks_lo) {
   static_assert(NKS == 4 || NKS == 1, "all of a tile's subtiles or one");
   const int lane = threadIdx.x & 63, n = lane & 15, g4 = lane >> 4;
   constexpr int PK = MfmaSmem<D, DV>::kPitchK;
@@ -348,13 +457,21 @@ __device__ __forceinline__ void attend_tile(WaveRows<D, DV, RB>& w, const MfmaSm
     // distance of the lane's key r of subtile ks: fd0 - (16 ks + r)
     const float fd0 = static_cast<float>(pos - j0 - 16 * ks_lo - 4 * g4);
     float mx = -INFINITY;
+    const float near = -w.ba[rb] * fd0;            // (Scaled) the linear bias of the lane's first key, sign included
 #pragma unroll
-    for (int ks = 0; ks < NKS; ++ks)
+    for (int ks = 0; ks < NKS; ++ks) {
+      f32x4v kscale = f32x4v{0.f, 0.f, 0.f, 0.f};
+      if (Scaled) kscale = *reinterpret_cast<const f32x4v*>(scales + 16 * (ks_lo + ks) + 4 * g4) * scale2;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        float sc = s[rb][ks][r] * scale2;
-        if (capped) sc = cap2 * tanh_fast(s[rb][ks][r] * cap_in);
-        if (bias) sc = fmaf(-w.ba[rb], __log2f(fmaf(w.bb[rb], fd0 - static_cast<float>(16 * ks + r), 1.f)), sc);
+        float sc;
+        if (Scaled) {
+          sc = fmaf(s[rb][ks][r], kscale[r], fmaf(w.ba[rb], static_cast<float>(16 * ks + r), near));
+        } else {
+          sc = s[rb][ks][r] * scale2;
+          if (capped) sc = cap2 * tanh_fast(s[rb][ks][r] * cap_in);
+          if (bias) sc = fmaf(-w.ba[rb], __log2f(fmaf(w.bb[rb], fd0 - static_cast<float>(16 * ks + r), 1.f)), sc);
+        }
         if (Masked) {
           const int j = j0 + 16 * (ks_lo + ks) + 4 * g4 + r;
           const int first = a.window_left >= 0 ? pos - a.window_left : 0;
@@ -363,6 +480,7 @@ __device__ __forceinline__ void attend_tile(WaveRows<D, DV, RB>& w, const MfmaSm
         s[rb][ks][r] = sc;
         mx = fmaxf(mx, sc);
       }
+    }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     const float m_new = fmaxf(w.m[rb], mx);
@@ -429,6 +547,22 @@ __device__ __forceinline__ void load_q(WaveRows<D, DV, RB>& w, int rb, const uin
     w.q[rb][st] = qrow ? __builtin_bit_cast(bf16x8, ld16g(qrow + 32 * st + 8 * g4)) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
 }
 
+// Whether every key of the tile from j0 on is visible to every query position in [p_lo, p_hi] / none of them to any.
+__device__ __forceinline__ bool tile_open(const hymeta_sink_attention_args& a, int j0, int p_lo, int p_hi) {
+  return j0 + kTileKeys - 1 <= p_lo && (a.window_left < 0 || j0 >= p_hi - a.window_left);
+}
+__device__ __forceinline__ bool tile_shut(const hymeta_sink_attention_args& a, int j0, int p_lo) {
+  return a.window_left >= 0 && j0 + kTileKeys - 1 < p_lo - a.window_left && j0 >= a.keep_first;
+}
+
+// The bias' constants of head h as attend_tile wants them.
+template <int D, int DV, int RB>
+__device__ __forceinline__ void load_bias(WaveRows<D, DV, RB>& w, int rb, const hymeta_sink_attention_args& a, int h) {
+  w.ba[rb] = a.bias_mode ? a.bias_a[h] : 0.f;
+  if (a.bias_mode == HYMETA_BIAS_LINEAR_DISTANCE) w.ba[rb] *= 1.4426950408889634f;
+  w.bb[rb] = a.bias_mode == HYMETA_BIAS_LOG_DISTANCE ? a.bias_b[h] : 0.f;
+}
+
 // Waves of a prompt workgroup: 8, or 4 for keys longer than 192 elements, whose query fragments (D / 8 registers) and
 // staging registers do not leave a wave of 8 its accumulators within 256 registers (408 bytes of scratch per lane at
 // 576; a workgroup of 4 waves has 512 registers per wave).
@@ -442,7 +576,9 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
   constexpr int kPrefillWaves = PrefillWaves<D>::value;
   constexpr int kRows = PrefillShape<RB, kPrefillWaves>::kRows;
   constexpr int kImages = 2 * sizeof(MfmaSmem<D, DV>) <= 159 * 1024 ? 2 : 1;        // (160 KB of LDS)
+  constexpr bool kScaled = Layout == HYMETA_KV_SCALED_KEY;
   __shared__ MfmaSmem<D, DV> sm[kImages];
+  __shared__ __attribute__((aligned(16))) float s_scale[kImages][kScaled ? kTileKeys : 4];
   const int s = blockIdx.z, h = blockIdx.y;
   const int row0 = a.query_start_loc[s];
   const int q = a.query_start_loc[s + 1] - row0;
@@ -458,8 +594,7 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
     const int r = wrow + 16 * rb + n;
     const bool ok = r < q;
     w.pos[rb] = ok ? ctx + r : -1;
-    w.ba[rb] = a.bias_mode ? a.bias_a[h] : 0.f;
-    w.bb[rb] = a.bias_mode ? a.bias_b[h] : 0.f;
+    load_bias<D, DV, RB>(w, rb, a, h);
     w.m[rb] = a.sink ? (a.sink_logits ? a.sink_logits[h] * 1.4426950408889634f : 0.f) : -INFINITY;
     w.l[rb] = (a.sink && g4 == 0) ? 1.f : 0.f;        // the sink's exp(m - m), counted once per row
     load_q<D, DV, RB>(w, rb, ok ? static_cast<const uint16_t*>(a.q) + static_cast<int64_t>(row0 + r) * a.q_stride_t + static_cast<int64_t>(h) * D : nullptr);
@@ -480,19 +615,19 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
   if (Layout == HYMETA_KV_VALUE_IN_KEY) stage.value_at = vs.first;
   if (Layout == HYMETA_KV_SHARED_KEY) stage.value_at = D + g * DV;
   stage.issue(a, bt, g, j_start, block_last);
-  stage.commit(sm[0]);
+  stage.commit(sm[0], s_scale[0]);
   if (kImages == 2 && next(j_start) <= block_last) stage.issue(a, bt, g, next(j_start), block_last);
   __syncthreads();
   if constexpr (kImages == 2) {
     int buf = 0;
     for (int j0 = j_start; j0 <= block_last; j0 = next(j0), buf ^= 1) {
       const int j1 = next(j0), j2 = next(j1);
-      if (j1 <= block_last) stage.commit(sm[buf ^ 1]);
+      if (j1 <= block_last) stage.commit(sm[buf ^ 1], s_scale[buf ^ 1]);
       if (j2 <= block_last) stage.issue(a, bt, g, j2, block_last);
-      if (wrow < q && j0 <= wave_last) {
-        // tiles wholly before the wave's first row (and no window) need no mask: every key is visible to every row
-        if (a.window_left < 0 && j0 + kTileKeys - 1 <= ctx + wrow) attend_tile<D, DV, RB, 4, false>(w, sm[buf], a, j0, 0);
-        else attend_tile<D, DV, RB, 4, true>(w, sm[buf], a, j0, 0);
+      if (wrow < q && j0 <= wave_last && !tile_shut(a, j0, ctx + wrow)) {
+        // tiles whose every key is visible to every row of the wave need no mask
+        if (tile_open(a, j0, ctx + wrow, wave_last)) attend_tile<D, DV, RB, 4, false, kScaled>(w, sm[buf], s_scale[buf], a, j0, 0);
+        else attend_tile<D, DV, RB, 4, true, kScaled>(w, sm[buf], s_scale[buf], a, j0, 0);
       }
       __syncthreads();
     }
@@ -502,13 +637,13 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
     for (int j0 = j_start; j0 <= block_last; j0 = next(j0)) {
       const bool more = next(j0) <= block_last;
       if (more) stage.issue(a, bt, g, next(j0), block_last);
-      if (wrow < q && j0 <= wave_last) {
-        if (a.window_left < 0 && j0 + kTileKeys - 1 <= ctx + wrow) attend_tile<D, DV, RB, 4, false>(w, sm[0], a, j0, 0);
-        else attend_tile<D, DV, RB, 4, true>(w, sm[0], a, j0, 0);
+      if (wrow < q && j0 <= wave_last && !tile_shut(a, j0, ctx + wrow)) {
+        if (tile_open(a, j0, ctx + wrow, wave_last)) attend_tile<D, DV, RB, 4, false, kScaled>(w, sm[0], s_scale[0], a, j0, 0);
+        else attend_tile<D, DV, RB, 4, true, kScaled>(w, sm[0], s_scale[0], a, j0, 0);
       }
       __syncthreads();
       if (more) {
-        stage.commit(sm[0]);
+        stage.commit(sm[0], s_scale[0]);
         __syncthreads();
       }
     }
@@ -525,7 +660,13 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
     uint16_t* out = static_cast<uint16_t*>(a.out) + (static_cast<int64_t>(row0 + r) * a.num_heads + h) * vs.total + vs.first;
 #pragma unroll
     for (int cb = 0; cb < DV / 16; ++cb) {
-      const f32x4v o = w.o[rb][cb] * inv;
+      f32x4v o = w.o[rb][cb] * inv;
+      if (a.elem_gate) {
+        float gate[4];
+        ActBf16::ld4(static_cast<const uint16_t*>(a.elem_gate) + static_cast<int64_t>(row0 + r) * a.elem_gate_stride_t + static_cast<int64_t>(h) * vs.total + vs.first + 16 * cb + 4 * g4, gate);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] *= ActBf16::sigmoid(gate[e]);
+      }
       *reinterpret_cast<u32x2*>(out + 16 * cb + 4 * g4) = u32x2{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
     }
   }
@@ -556,7 +697,9 @@ struct DecodeMerge {
 template <int D, int DV, int RB, int Layout>
 __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_kernel(hymeta_sink_attention_args a, int splits, int tiles_per_split, ValueSlice vs) {
   constexpr int kImages = DecodeImages<D, DV>::value;
+  constexpr bool kScaled = Layout == HYMETA_KV_SCALED_KEY;
   __shared__ MfmaSmem<D, DV> sm[kImages];
+  __shared__ __attribute__((aligned(16))) float s_scale[kImages][kScaled ? kTileKeys : 4];
   int s = blockIdx.z, g = blockIdx.y, split = blockIdx.x;
   if (Layout == HYMETA_KV_SHARED_KEY) {
     // The value groups of a (sequence, split) read the same key tiles.  Workgroups go to the chip's 8 dies (each with an
@@ -597,8 +740,7 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
     const bool ok = r < HG;
     const int h = g * group + vs.h_first + (ok ? r : 0);
     w.pos[rb] = ok ? pos : -1;
-    w.ba[rb] = a.bias_mode ? a.bias_a[h] : 0.f;
-    w.bb[rb] = a.bias_mode ? a.bias_b[h] : 0.f;
+    load_bias<D, DV, RB>(w, rb, a, h);
     w.m[rb] = -INFINITY;
     w.l[rb] = 0.f;
     load_q<D, DV, RB>(w, rb, ok ? static_cast<const uint16_t*>(a.q) + static_cast<int64_t>(t) * a.q_stride_t + static_cast<int64_t>(h) * D : nullptr);
@@ -610,7 +752,7 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
   if (Layout == HYMETA_KV_SHARED_KEY) stage.value_at = D + g * DV;
   if (v_lo <= v_hi) {
     stage.issue(a, bt, g, tile(v_lo), pos);
-    stage.commit(sm[0]);
+    stage.commit(sm[0], s_scale[0]);
     if (kImages == 2 && v_lo + 1 <= v_hi) stage.issue(a, bt, g, tile(v_lo + 1), pos);
   }
   __syncthreads();
@@ -618,11 +760,11 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
     int buf = 0;
     for (int v = v_lo; v <= v_hi; ++v, buf ^= 1) {
       const int j0 = tile(v);
-      if (v + 1 <= v_hi) stage.commit(sm[buf ^ 1]);
+      if (v + 1 <= v_hi) stage.commit(sm[buf ^ 1], s_scale[buf ^ 1]);
       if (v + 2 <= v_hi) stage.issue(a, bt, g, tile(v + 2), pos);
       if (j0 + 16 * wave <= pos) {
-        if (a.window_left < 0 && j0 + kTileKeys - 1 <= pos) attend_tile<D, DV, RB, 1, false>(w, sm[buf], a, j0, wave);
-        else attend_tile<D, DV, RB, 1, true>(w, sm[buf], a, j0, wave);
+        if (tile_open(a, j0, pos, pos)) attend_tile<D, DV, RB, 1, false, kScaled>(w, sm[buf], s_scale[buf], a, j0, wave);
+        else attend_tile<D, DV, RB, 1, true, kScaled>(w, sm[buf], s_scale[buf], a, j0, wave);
       }
       __syncthreads();
     }
@@ -633,12 +775,12 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
       const bool more = v + 1 <= v_hi;
       if (more) stage.issue(a, bt, g, tile(v + 1), pos);
       if (j0 + 16 * wave <= pos) {
-        if (a.window_left < 0 && j0 + kTileKeys - 1 <= pos) attend_tile<D, DV, RB, 1, false>(w, sm[0], a, j0, wave);
-        else attend_tile<D, DV, RB, 1, true>(w, sm[0], a, j0, wave);
+        if (tile_open(a, j0, pos, pos)) attend_tile<D, DV, RB, 1, false, kScaled>(w, sm[0], s_scale[0], a, j0, wave);
+        else attend_tile<D, DV, RB, 1, true, kScaled>(w, sm[0], s_scale[0], a, j0, wave);
       }
       __syncthreads();
       if (more) {
-        stage.commit(sm[0]);
+        stage.commit(sm[0], s_scale[0]);
         __syncthreads();
       }
     }
@@ -726,7 +868,10 @@ __global__ __launch_bounds__(64) void sink_attention_decode_combine_kernel(hymet
       const float ms = base[sp * stride + DV];
       if (ms != -INFINITY) acc += base[sp * stride + c] * __builtin_amdgcn_exp2f(ms - m);
     }
-    out[c] = f2bf(acc * inv);
+    acc *= inv;
+    if (a.elem_gate)
+      acc *= ActBf16::sigmoid(bf2f(static_cast<const uint16_t*>(a.elem_gate)[static_cast<int64_t>(t) * a.elem_gate_stride_t + static_cast<int64_t>(h) * vs.total + vs.first + c]));
+    out[c] = f2bf(acc);
   }
 }
 
@@ -742,13 +887,24 @@ inline bool mfma_shape(const hymeta_sink_attention_args& a) {
   // one key for all heads: the concatenated keys of 1 / 2 / 4 / 8 key/value heads of 64 or 128
   if (a.kv_layout == HYMETA_KV_SHARED_KEY)
     dims = (a.head_dim == 64 || a.head_dim == 128 || a.head_dim == 256 || a.head_dim == 512) && (a.v_dim == 64 || a.v_dim == 128);
+  // key and value in one vector
+  if (a.kv_layout == HYMETA_KV_SCALED_KEY)
+    dims = a.head_dim == a.v_dim && (a.head_dim == 32 || a.head_dim == 64 || a.head_dim == 96 || a.head_dim == 128) &&
+           a.bias_mode != HYMETA_BIAS_LOG_DISTANCE && a.softcap <= 0.f;
+  else if (a.bias_mode == HYMETA_BIAS_LINEAR_DISTANCE) dims = false;
+  if (a.elem_gate && (a.elem_gate_stride_t % 4 != 0 || reinterpret_cast<uintptr_t>(a.elem_gate) % 8 != 0)) dims = false;
   return a.act_dtype == HYMETA_BF16 && dims && a.q_stride_t % 8 == 0 &&
          (a.block_size & (a.block_size - 1)) == 0 &&
          (reinterpret_cast<uintptr_t>(a.q) | reinterpret_cast<uintptr_t>(a.kv_cache) | reinterpret_cast<uintptr_t>(a.out)) % 16 == 0;
 }
 
-inline int decode_splits(int num_seqs, int num_heads, int num_kv_heads, int max_seq_len) {
-  const int tiles = (max_seq_len + kTileKeys - 1) / kTileKeys;
+// window_left >= 0: a row reads the kept first keys' tiles and the window's, however long the sequence is.
+inline int decode_splits(int num_seqs, int num_heads, int num_kv_heads, int max_seq_len, int window_left = -1, int keep_first = 0) {
+  int tiles = (max_seq_len + kTileKeys - 1) / kTileKeys;
+  if (window_left >= 0) {
+    const int64_t seen = (static_cast<int64_t>(keep_first) + kTileKeys - 1) / kTileKeys + static_cast<int64_t>(window_left) / kTileKeys + 2;
+    if (seen < tiles) tiles = static_cast<int>(seen);
+  }
   // Workgroups aimed at: a workgroup's fixed cost (query fragments, first tile, the merge of its waves, its partial) grows
   // with the query heads it carries, so fewer, longer workgroups pay.  Measured at 64 sequences x 4096 keys: 28 heads on
   // one row of 192: 93 / 67 / 56 / 87 us at 1024 / 512 / 256 / 128; 16 heads on it: 53 / 40 / 45; 4 key/value heads with
@@ -768,7 +924,7 @@ int launch_mfma(const hymeta_sink_attention_args& a, hipStream_t st, ValueSlice 
     hipLaunchKernelGGL((sink_attention_prefill_mfma_kernel<D, DV, kRB, Layout>), grid, dim3(64 * PrefillWaves<D>::value), 0, st, a, vs);
   }
   // sequences with a single row: every step but a pure prompt step has some; a prompt of one token is one too
-  const int splits = decode_splits(a.num_seqs, a.num_heads, a.num_kv_heads, a.max_seq_len);
+  const int splits = decode_splits(a.num_seqs, a.num_heads, a.num_kv_heads, a.max_seq_len, a.window_left, a.keep_first);
   const int tiles = (a.max_seq_len + kTileKeys - 1) / kTileKeys;
   const int tiles_per_split = (tiles + splits - 1) / splits;
   const dim3 grid = Layout == HYMETA_KV_SHARED_KEY ? dim3((splits * a.num_seqs + 7) / 8 * 8 * a.num_kv_heads) : dim3(splits, a.num_kv_heads, a.num_seqs);
@@ -812,6 +968,35 @@ extern "C" int hymeta_qk_norm_cache(const hymeta_qk_norm_cache_args* args, hymet
   return launch_status();
 }
 
+extern "C" int hymeta_scaled_key_cache(const hymeta_scaled_key_cache_args* args, hymeta_stream_t stream) {
+  if (!args_ok(args)) return HYMETA_ERR_INVALID_ARG;
+  const hymeta_scaled_key_cache_args& a = *args;
+  if (a.num_tokens < 0 || a.num_heads <= 0 || a.num_kv_heads <= 0 || a.head_dim <= 0 || a.num_blocks < 0) return HYMETA_ERR_INVALID_ARG;
+  if (!act_dtype_ok(a.act_dtype)) return HYMETA_ERR_UNSUPPORTED;
+  if (a.num_tokens == 0) return HYMETA_OK;
+  if (!a.qk || !a.q_weight || !a.k_weight || a.qk_stride_t < static_cast<int64_t>(a.num_heads + a.num_kv_heads) * a.head_dim) return HYMETA_ERR_INVALID_ARG;
+  if (a.slot_mapping && (!a.kv_cache || a.block_size <= 0 || reinterpret_cast<uintptr_t>(a.kv_cache) % 16 != 0)) return HYMETA_ERR_INVALID_ARG;
+  if (a.temp_coef != 0.f && (!a.positions || !(a.temp_every > 0.0))) return HYMETA_ERR_INVALID_ARG;
+  hipStream_t st = begin_launches(stream);
+  const int bytes = a.act_dtype == HYMETA_BF16 ? 2 : 4;
+  // four elements a lane where a head and a row are whole fours and a head fits a wave
+  const bool vec = a.head_dim % 4 == 0 && a.head_dim <= 256 && a.qk_stride_t % 4 == 0 && reinterpret_cast<uintptr_t>(a.qk) % (4 * bytes) == 0;
+  int lanes = 64;
+  if (vec) {
+    lanes = 1;
+    while (4 * lanes < a.head_dim) lanes *= 2;
+  }
+  const dim3 grid(a.num_tokens), block(256);
+  if (a.act_dtype == HYMETA_BF16) {
+    if (vec) hipLaunchKernelGGL((scaled_key_cache_kernel<ActBf16, true>), grid, block, 0, st, a, lanes);
+    else hipLaunchKernelGGL((scaled_key_cache_kernel<ActBf16, false>), grid, block, 0, st, a, lanes);
+  } else {
+    if (vec) hipLaunchKernelGGL((scaled_key_cache_kernel<ActF32, true>), grid, block, 0, st, a, lanes);
+    else hipLaunchKernelGGL((scaled_key_cache_kernel<ActF32, false>), grid, block, 0, st, a, lanes);
+  }
+  return launch_status();
+}
+
 extern "C" size_t hymeta_sink_attention_workspace_bytes(int32_t num_seqs, int32_t num_heads, int32_t num_kv_heads, int32_t v_dim,
                                                         int32_t max_seq_len) {
   if (num_seqs <= 0 || num_heads <= 0 || num_kv_heads <= 0 || v_dim <= 0) return 0;
@@ -828,13 +1013,15 @@ extern "C" int hymeta_sink_attention(const hymeta_sink_attention_args* args, hym
   if (a.num_heads % a.num_kv_heads != 0) return HYMETA_ERR_INVALID_ARG;
   if (!act_dtype_ok(a.act_dtype)) return HYMETA_ERR_UNSUPPORTED;
   if (a.head_dim > kMaxHeadDim || a.v_dim > 64 * kMaxVChunks) return HYMETA_ERR_UNSUPPORTED;
-  if (a.bias_mode != HYMETA_BIAS_NONE && a.bias_mode != HYMETA_BIAS_LOG_DISTANCE) return HYMETA_ERR_UNSUPPORTED;
-  if (a.kv_layout != HYMETA_KV_KEY_THEN_VALUE && a.kv_layout != HYMETA_KV_VALUE_IN_KEY && a.kv_layout != HYMETA_KV_SHARED_KEY) return HYMETA_ERR_UNSUPPORTED;
+  if (a.bias_mode < HYMETA_BIAS_NONE || a.bias_mode > HYMETA_BIAS_LINEAR_DISTANCE) return HYMETA_ERR_UNSUPPORTED;
+  if (a.kv_layout < HYMETA_KV_KEY_THEN_VALUE || a.kv_layout > HYMETA_KV_SCALED_KEY) return HYMETA_ERR_UNSUPPORTED;
+  if (a.kv_layout == HYMETA_KV_SCALED_KEY && (a.v_dim != a.head_dim || reinterpret_cast<uintptr_t>(a.kv_cache) % 16 != 0)) return HYMETA_ERR_INVALID_ARG;
   if (a.window_left >= 0 && a.keep_first < 0) return HYMETA_ERR_INVALID_ARG;
   if (a.kv_layout == HYMETA_KV_VALUE_IN_KEY && a.v_dim > a.head_dim) return HYMETA_ERR_INVALID_ARG;
   if (a.num_tokens == 0 || a.num_seqs == 0) return HYMETA_OK;
   if (!a.q || !a.kv_cache || !a.out || !a.block_tables || !a.query_start_loc || !a.seq_lens) return HYMETA_ERR_INVALID_ARG;
-  if (a.bias_mode != HYMETA_BIAS_NONE && (!a.bias_a || !a.bias_b)) return HYMETA_ERR_INVALID_ARG;
+  if (a.bias_mode != HYMETA_BIAS_NONE && (!a.bias_a || (a.bias_mode == HYMETA_BIAS_LOG_DISTANCE && !a.bias_b))) return HYMETA_ERR_INVALID_ARG;
+  if (a.elem_gate && a.elem_gate_stride_t < static_cast<int64_t>(a.num_heads) * a.v_dim) return HYMETA_ERR_INVALID_ARG;
   if (a.softcap < 0.f || (a.head_gate && a.head_gate_stride_t < a.num_heads)) return HYMETA_ERR_INVALID_ARG;
   if (a.num_heads > 65535) return HYMETA_ERR_UNSUPPORTED;
   hipStream_t st = begin_launches(stream);
@@ -854,6 +1041,11 @@ extern "C" int hymeta_sink_attention(const hymeta_sink_attention_args* args, hym
         if (rc != HYMETA_OK) return rc;
       }
       return HYMETA_OK;
+    }
+    if (a.kv_layout == HYMETA_KV_SCALED_KEY) {
+      constexpr int kScaled = HYMETA_KV_SCALED_KEY;
+      return a.head_dim == 32 ? launch_mfma<32, 32, kScaled>(a, st) : a.head_dim == 64 ? launch_mfma<64, 64, kScaled>(a, st)
+           : a.head_dim == 96 ? launch_mfma<96, 96, kScaled>(a, st) : launch_mfma<128, 128, kScaled>(a, st);
     }
     if (a.kv_layout == HYMETA_KV_SHARED_KEY) {
       constexpr int kShared = HYMETA_KV_SHARED_KEY;

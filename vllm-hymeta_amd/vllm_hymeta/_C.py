@@ -26,20 +26,23 @@ GATE_70B_LOWER_BOUND = 3
 
 BIAS_NONE = 0
 BIAS_LOG_DISTANCE = 1
+BIAS_LINEAR_DISTANCE = 2
 KV_KEY_THEN_VALUE = 0
 KV_VALUE_IN_KEY = 1
 KV_SHARED_KEY = 2
+KV_SCALED_KEY = 3
 GLU_NONE, GLU_SILU, GLU_CLAMPED, GLU_RELU2 = 0, 1, 2, 3
-ACT_CLAMPED_GLU, ACT_XIELU, ACT_SIGMOID_MUL, ACT_SILU_MUL, ACT_RELU2 = 0, 1, 2, 3, 4
+ACT_CLAMPED_GLU, ACT_XIELU, ACT_SIGMOID_MUL, ACT_SILU_MUL, ACT_RELU2, ACT_GELU_MUL, ACT_GELU_ROWS = 0, 1, 2, 3, 4, 5, 6
 ROUTE_SIGMOID_SUM, ROUTE_SOFTMAX_CHOSEN, ROUTE_SOFTMAX_GROUPED = 0, 1, 2
 GATE_SIGMOID, GATE_SILU = 0, 1
 STREAM_MAX_TERMS = 6
 SCAN_CHUNK = 64
+DELTA_CHUNK = 64
 MAX_STREAMS = 16
 LIGHTNING_CHUNK = 64
 CONV_MAX_TAPS = 8
 
-ABI_VERSION = 7
+ABI_VERSION = 8
 ERR_SCRATCH_LIMIT = -5
 GEMM_TICKET_BYTES = 16384
 STATIC_SCRATCH_BYTES = 16 << 20
@@ -307,7 +310,7 @@ class EmbedRowsArgs(_Args):
         _SIZE,
         ("token_ids", _ptr), ("table", _ptr), ("add", _ptr), ("out", _ptr),
         ("num_tokens", _i32), ("width", _i32), ("vocab", _i32), ("act_dtype", _i32),
-        ("scale", _f32),
+        ("scale", _f32), ("positions", _ptr), ("pos_freqs", _ptr), ("h_out", _ptr),
     ]
 
 
@@ -328,7 +331,7 @@ class NormResidualArgs(_Args):
         ("y", _ptr), ("weight", _ptr), ("post_add", _ptr), ("x", _ptr),
         ("num_tokens", _i32), ("width", _i32), ("act_dtype", _i32),
         ("eps", _f32), ("weight_offset", _f32), ("mult", _f32),
-        ("y_stride_t", _i64), ("x_stride_t", _i64),
+        ("y_stride_t", _i64), ("x_stride_t", _i64), ("h_out", _ptr),
     ]
 
 
@@ -365,6 +368,7 @@ class SinkAttentionArgs(_Args):
         ("num_blocks", _i64), ("q_stride_t", _i64), ("block_table_stride", _i64),
         ("sink_logits", _ptr), ("kv_layout", _i32), ("keep_first", _i32),
         ("softcap", _f32), ("head_gate", _ptr), ("head_gate_stride_t", _i64),
+        ("elem_gate", _ptr), ("elem_gate_stride_t", _i64),
     ]
 
 
@@ -470,6 +474,7 @@ class ActivationArgs(_Args):
         ("kind", _i32), ("num_rows", _i32), ("n", _i32), ("act_dtype", _i32),
         ("p0", _f32), ("p1", _f32),
         ("x_stride", _i64), ("gate_stride", _i64), ("out_stride", _i64),
+        ("gate_rows", _ptr), ("gate_row_count", _i64),
     ]
 
 
@@ -569,6 +574,30 @@ class DecayScanArgs(_Args):
     ]
 
 
+class ScaledKeyCacheArgs(_Args):
+    _fields_ = [
+        _SIZE,
+        ("qk", _ptr), ("q_weight", _ptr), ("k_weight", _ptr), ("kv_cache", _ptr), ("slot_mapping", _ptr), ("positions", _ptr),
+        ("temp_every", C.c_double),
+        ("num_tokens", _i32), ("num_heads", _i32), ("num_kv_heads", _i32), ("head_dim", _i32), ("block_size", _i32), ("act_dtype", _i32),
+        ("eps", _f32), ("temp_coef", _f32),
+        ("num_blocks", _i64), ("qk_stride_t", _i64),
+    ]
+
+
+class DeltaRuleArgs(_Args):
+    _fields_ = [
+        _SIZE,
+        ("q", _ptr), ("k", _ptr), ("v", _ptr), ("beta_logit", _ptr), ("log2_decay", _ptr), ("state", _ptr), ("out", _ptr),
+        ("norm_weight", _ptr), ("gate", _ptr), ("query_start_loc", _ptr), ("context_lens", _ptr), ("slot_idx", _ptr),
+        ("num_tokens", _i32), ("num_seqs", _i32), ("num_heads", _i32), ("num_qk_heads", _i32), ("head_dim", _i32), ("v_dim", _i32),
+        ("act_dtype", _i32), ("max_query_len", _i32),
+        ("q_scale", _f32), ("unit_eps", _f32), ("norm_eps", _f32),
+        ("q_stride_t", _i64), ("k_stride_t", _i64), ("v_stride_t", _i64), ("beta_stride_t", _i64), ("gate_stride_t", _i64),
+        ("workspace", _ptr), ("workspace_bytes", _sz),
+    ]
+
+
 _SIGNATURES = {
     "hymeta_strerror": (C.c_char_p, [C.c_int]),
     "hymeta_abi_version": (C.c_int, []),
@@ -664,6 +693,9 @@ _SIGNATURES = {
     "hymeta_causal_conv": (C.c_int, [C.POINTER(CausalConvArgs), _ptr]),
     "hymeta_decay_scan_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32]),
     "hymeta_decay_scan": (C.c_int, [C.POINTER(DecayScanArgs), _ptr]),
+    "hymeta_scaled_key_cache": (C.c_int, [C.POINTER(ScaledKeyCacheArgs), _ptr]),
+    "hymeta_delta_rule_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32]),
+    "hymeta_delta_rule": (C.c_int, [C.POINTER(DeltaRuleArgs), _ptr]),
 }
 
 STRUCTS = {
@@ -709,6 +741,8 @@ STRUCTS = {
     "hymeta_rotary_cache_args": RotaryCacheArgs,
     "hymeta_causal_conv_args": CausalConvArgs,
     "hymeta_decay_scan_args": DecayScanArgs,
+    "hymeta_scaled_key_cache_args": ScaledKeyCacheArgs,
+    "hymeta_delta_rule_args": DeltaRuleArgs,
 }
 
 

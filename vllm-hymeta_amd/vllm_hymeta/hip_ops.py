@@ -1476,9 +1476,12 @@ def _i32vec(t: torch.Tensor, n: int, name: str) -> None:
     _require(t.dtype == torch.int32 and t.is_contiguous() and t.numel() >= n, f"{name} must be contiguous int32 [{n}]")
 
 
-def embed_rows(token_ids: torch.Tensor, table: torch.Tensor, add: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
-    """fp32 ``[T, W]`` rows ``table[token_ids] * scale (+ add)``: the start of an fp32 residual stream."""
-    _dev(token_ids, table, add)
+def embed_rows(token_ids: torch.Tensor, table: torch.Tensor, add: Optional[torch.Tensor] = None, scale: float = 1.0,
+               positions: Optional[torch.Tensor] = None, pos_freqs: Optional[torch.Tensor] = None, copy: bool = False):
+    """fp32 ``[T, W]`` rows ``table[token_ids] * scale (+ add)``: the start of an fp32 residual stream.  With ``pos_freqs``
+    (float64, one per pair of columns) ``sin(p f_i)`` is added to column ``2 i`` and ``cos(p f_i)`` to column ``2 i + 1`` at
+    position ``p`` (``positions`` int64).  ``copy``: returns ``(rows, rows rounded to the table's type)``."""
+    _dev(token_ids, table, add, positions, pos_freqs)
     _require(token_ids.dtype == torch.int64 and token_ids.dim() == 1 and token_ids.is_contiguous(), "token_ids must be contiguous int64 [T]")
     _require(table.dim() == 2 and table.is_contiguous(), "table must be contiguous [vocab, width]")
     V, W = table.shape
@@ -1487,8 +1490,16 @@ def embed_rows(token_ids: torch.Tensor, table: torch.Tensor, add: Optional[torch
     a = _C.EmbedRowsArgs()
     a.token_ids, a.table, a.add, a.out = _p(token_ids), _p(table), _p(add), _p(out)
     a.num_tokens, a.width, a.vocab, a.act_dtype, a.scale = token_ids.shape[0], W, V, _act(table), float(scale)
+    if pos_freqs is not None:
+        _require(pos_freqs.dtype == torch.float64 and pos_freqs.is_contiguous() and pos_freqs.numel() == (W + 1) // 2,
+                 "pos_freqs must be contiguous float64, one per pair of columns")
+        _require(positions is not None and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == token_ids.numel(),
+                 "positions must be int64 [T]")
+        a.positions, a.pos_freqs = _p(positions), _p(pos_freqs)
+    h = torch.empty(token_ids.shape[0], W, dtype=table.dtype, device=table.device) if copy else None
+    a.h_out = _p(h)
     _C.check(_C.load().hymeta_embed_rows(C.byref(a), _stream(table)), "hymeta_embed_rows")
-    return out
+    return (out, h) if copy else out
 
 
 def norm_conv(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype, weight_offset: float = 0.0,
@@ -1531,8 +1542,9 @@ def norm_conv(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torc
 
 
 def norm_residual_(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, mult: float = 1.0,
-                   weight_offset: float = 0.0, post_add: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``x += mult * rmsnorm(y) * (weight_offset + weight) (+ post_add)`` on the fp32 rows ``x [T, W]``, in place."""
+                   weight_offset: float = 0.0, post_add: Optional[torch.Tensor] = None, copy: bool = False) -> torch.Tensor:
+    """``x += mult * rmsnorm(y) * (weight_offset + weight) (+ post_add)`` on the fp32 rows ``x [T, W]``, in place.  Returns
+    ``x``, or with ``copy`` its new rows rounded to y's type."""
     _dev(x, y, weight, post_add)
     _require(x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1, "x must be row-contiguous fp32 [T, W]")
     T, W = x.shape
@@ -1543,8 +1555,10 @@ def norm_residual_(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: 
     a.y, a.weight, a.post_add, a.x = _p(y), _p(weight), _p(post_add), _p(x)
     a.num_tokens, a.width, a.act_dtype = T, W, _act(y)
     a.eps, a.weight_offset, a.mult, a.y_stride_t, a.x_stride_t = eps, weight_offset, mult, y.stride(0), x.stride(0)
+    h = torch.empty(T, W, dtype=y.dtype, device=x.device) if copy else None
+    a.h_out = _p(h)
     _C.check(_C.load().hymeta_norm_residual(C.byref(a), _stream(x)), "hymeta_norm_residual")
-    return x
+    return x if h is None else h
 
 
 def mingru(zug: torch.Tensor, state: torch.Tensor, query_start_loc: torch.Tensor, context_lens: torch.Tensor,
@@ -1596,24 +1610,68 @@ def qk_norm_cache_(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
     _C.check(_C.load().hymeta_qk_norm_cache(C.byref(a), _stream(qkv)), "hymeta_qk_norm_cache")
 
 
+def scaled_key_row(num_kv_heads: int, head_dim: int, dtype: torch.dtype) -> int:
+    """Elements of a ``scaled_key`` cache row: a vector per key/value head, then (from the next multiple of 4 bytes on) an
+    fp32 factor per head, padded to 16 bytes."""
+    size = torch.empty(0, dtype=dtype).element_size()
+    at = (num_kv_heads * head_dim * size + 3) // 4 * 4
+    return (at + 4 * num_kv_heads + 15) // 16 * 16 // size
+
+
+def scaled_key_cache_(qk: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, q_weight: torch.Tensor, k_weight: torch.Tensor,
+                      eps: float, kv_cache: Optional[torch.Tensor] = None, slot_mapping: Optional[torch.Tensor] = None,
+                      temp_coef: float = 0.0, temp_every: float = 1.0, positions: Optional[torch.Tensor] = None) -> None:
+    """On the rows ``qk [T, H D + G D (+ ...)]`` of a fused projection: queries, in place, become ``rmsnorm(q) * q_weight *
+    k_weight`` times ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)`` at position ``p`` (``positions`` int64); the cache
+    ``[blocks, block_size, 1, scaled_key_row(G, D)]`` gets at ``slot_mapping`` the keys as they are and their inverse root mean
+    squares, so that the product of a query with a stored key times its factor is that of the normed query and key."""
+    _dev(qk, q_weight, k_weight, kv_cache, slot_mapping, positions)
+    T = qk.shape[0]
+    H, G, D = num_heads, num_kv_heads, head_dim
+    _require(qk.dim() == 2 and qk.stride(1) == 1 and qk.shape[1] >= (H + G) * D, "qk must be row-contiguous [T, H D + G D (+ ...)]")
+    _require(q_weight is not None and k_weight is not None, "both norms' weights")
+    _f32vec(q_weight, D, "q_weight")
+    _f32vec(k_weight, D, "k_weight")
+    a = _C.ScaledKeyCacheArgs()
+    a.qk, a.q_weight, a.k_weight = _p(qk), _p(q_weight), _p(k_weight)
+    a.num_tokens, a.num_heads, a.num_kv_heads, a.head_dim, a.act_dtype = T, H, G, D, _act(qk)
+    a.eps, a.temp_coef, a.temp_every, a.qk_stride_t, a.block_size = eps, float(temp_coef), float(temp_every), qk.stride(0), 1
+    if temp_coef:
+        _require(positions is not None and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == T, "positions must be int64 [T]")
+        _require(temp_every > 0, "temp_every counts tokens")
+        a.positions = _p(positions)
+    if kv_cache is not None and kv_cache.numel() > 0 and slot_mapping is not None:
+        _require(kv_cache.dtype == qk.dtype and kv_cache.is_contiguous() and kv_cache.dim() == 4 and kv_cache.shape[2:] == (1, scaled_key_row(G, D, qk.dtype)),
+                 "kv_cache must be contiguous [blocks, block_size, 1, scaled_key_row(G, D)]")
+        _require(slot_mapping.dtype == torch.int64 and slot_mapping.is_contiguous() and slot_mapping.numel() == T, "slot_mapping must be int64 [T]")
+        a.kv_cache, a.slot_mapping, a.num_blocks, a.block_size = _p(kv_cache), _p(slot_mapping), kv_cache.shape[0], kv_cache.shape[1]
+    _C.check(_C.load().hymeta_scaled_key_cache(C.byref(a), _stream(qk)), "hymeta_scaled_key_cache")
+
+
 def sink_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_tables: torch.Tensor, query_start_loc: torch.Tensor,
                    seq_lens: torch.Tensor, num_kv_heads: int, head_dim: int, v_dim: int, scale: float,
                    max_query_len: int, max_seq_len: int, bias_a: Optional[torch.Tensor] = None,
                    bias_b: Optional[torch.Tensor] = None, sink: bool = True, window_left: int = -1,
                    sink_logits: Optional[torch.Tensor] = None, value_in_key: bool = False, shared_key: bool = False,
-                   keep_first: int = 0, softcap: float = 0.0, head_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   keep_first: int = 0, softcap: float = 0.0, head_gate: Optional[torch.Tensor] = None, scaled_key: bool = False,
+                   slopes: Optional[torch.Tensor] = None, elem_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention of the rows ``q [T, H, D]`` over their sequences' paged keys (this step's included):
     ``softmax`` over ``scale q.k - bias_a[h] ln(1 + bias_b[h] (i - j))`` with, for ``sink``, ``exp(sink_logits[h])`` (one
     without ``sink_logits``) added to the denominator.  ``softcap > 0``: ``scale q.k`` becomes ``softcap tanh(scale q.k /
-    softcap)``.  ``head_gate [T, H]`` (a view with any row stride): head ``h``'s output is multiplied by its sigmoid.  ``value_in_key``: a cache row holds ``D`` elements per key/value
+    softcap)``.  ``head_gate [T, H]`` (a view with any row stride): head ``h``'s output is multiplied by its sigmoid;
+    ``elem_gate [T, H Dv]``: the output is multiplied by its sigmoid element by element.  ``slopes [H]`` (in place of ``bias_a`` /
+    ``bias_b``): the bias is ``slopes[h] (i - j)``.  ``scaled_key``: cache rows as ``scaled_key_cache_`` writes them.  ``value_in_key``: a cache row holds ``D`` elements per key/value
     head, the first ``Dv`` of which are also the value (a latent that keys and values share).  Returns ``[T, H, Dv]``."""
-    _dev(q, kv_cache, block_tables, query_start_loc, seq_lens, bias_a, bias_b, sink_logits)
+    _dev(q, kv_cache, block_tables, query_start_loc, seq_lens, bias_a, bias_b, sink_logits, slopes, elem_gate)
     _require(q.dim() == 3 and q.stride(2) == 1 and q.stride(1) == head_dim and q.shape[2] == head_dim, "q must be [T, H, D] with contiguous heads")
     T, H, _ = q.shape
     row = head_dim if value_in_key else head_dim + v_dim
     _require(not value_in_key or v_dim <= head_dim, "a value inside its key cannot be longer than the key")
-    _require(not (value_in_key and shared_key), "one row layout at a time")
+    _require(int(value_in_key) + int(shared_key) + int(scaled_key) <= 1, "one row layout at a time")
     cache_tail = (1, head_dim + num_kv_heads * v_dim) if shared_key else (num_kv_heads, row)
+    if scaled_key:
+        _require(v_dim == head_dim, "a scaled key is its value")
+        cache_tail = (1, scaled_key_row(num_kv_heads, head_dim, q.dtype))
     _require(kv_cache.dtype == q.dtype and kv_cache.is_contiguous() and kv_cache.dim() == 4
              and kv_cache.shape[2:] == cache_tail, f"kv_cache must be contiguous [blocks, block_size, {cache_tail[0]}, {cache_tail[1]}]")
     _require(keep_first >= 0, "keep_first counts tokens")
@@ -1626,6 +1684,8 @@ def sink_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_tables: torch.
     _require((bias_a is None) == (bias_b is None), "bias_a and bias_b come together")
     _f32vec(bias_a, H, "bias_a")
     _f32vec(bias_b, H, "bias_b")
+    _f32vec(slopes, H, "slopes")
+    _require(slopes is None or bias_a is None, "one distance bias at a time")
     out = torch.empty(T, H, v_dim, dtype=q.dtype, device=q.device)
     lib = _C.load()
     a = _C.SinkAttentionArgs()
@@ -1638,13 +1698,19 @@ def sink_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_tables: torch.
     a.num_tokens, a.num_seqs, a.num_heads, a.num_kv_heads, a.head_dim, a.v_dim = T, S, H, num_kv_heads, head_dim, v_dim
     a.block_size, a.act_dtype, a.num_blocks = kv_cache.shape[1], _act(q), kv_cache.shape[0]
     a.bias_mode = _C.BIAS_NONE if bias_a is None else _C.BIAS_LOG_DISTANCE
+    if slopes is not None:
+        a.bias_mode, a.bias_a = _C.BIAS_LINEAR_DISTANCE, _p(slopes)
+    if elem_gate is not None:
+        _require(elem_gate.shape == (T, H * v_dim) and elem_gate.stride(1) == 1 and elem_gate.dtype == q.dtype, "elem_gate must be [T, H Dv] of q's type with contiguous rows")
+        a.elem_gate, a.elem_gate_stride_t = _p(elem_gate), elem_gate.stride(0)
     a.sink, a.window_left, a.max_query_len, a.max_seq_len, a.scale = int(bool(sink)), window_left, max_query_len, max_seq_len, scale
     a.sink_logits, a.keep_first, a.softcap = _p(sink_logits), keep_first, float(softcap)
     if head_gate is not None:
         _dev(q, head_gate)
         _require(head_gate.shape == (T, H) and head_gate.stride(1) == 1 and head_gate.dtype == q.dtype, "head_gate must be [T, H] of q's type with contiguous heads")
         a.head_gate, a.head_gate_stride_t = _p(head_gate), head_gate.stride(0)
-    a.kv_layout = _C.KV_SHARED_KEY if shared_key else (_C.KV_VALUE_IN_KEY if value_in_key else _C.KV_KEY_THEN_VALUE)
+    a.kv_layout = (_C.KV_SCALED_KEY if scaled_key else _C.KV_SHARED_KEY if shared_key else
+                   _C.KV_VALUE_IN_KEY if value_in_key else _C.KV_KEY_THEN_VALUE)
     a.q_stride_t, a.block_table_stride = q.stride(0), block_tables.stride(0)
     _C.check(lib.hymeta_sink_attention(C.byref(a), _stream(q)), "hymeta_sink_attention")
     return out
@@ -1898,8 +1964,9 @@ def gated_rms_norm(x: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.T
 
 
 def _activation(kind: int, x: torch.Tensor, n: int, p0: float, p1: float, gate: Optional[torch.Tensor] = None,
-                out: Optional[torch.Tensor] = None, num_rows_dev: Optional[torch.Tensor] = None) -> torch.Tensor:
-    _dev(x, gate, out, num_rows_dev)
+                out: Optional[torch.Tensor] = None, num_rows_dev: Optional[torch.Tensor] = None,
+                gate_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    _dev(x, gate, out, num_rows_dev, gate_rows)
     _require(x.dim() == 2 and x.stride(1) == 1, "x must be row-contiguous")
     rows = x.shape[0]
     if out is None:
@@ -1909,6 +1976,8 @@ def _activation(kind: int, x: torch.Tensor, n: int, p0: float, p1: float, gate: 
     a.x, a.gate, a.out, a.num_rows_dev = _p(x), _p(gate), _p(out), _p(num_rows_dev)
     a.kind, a.num_rows, a.n, a.act_dtype, a.p0, a.p1 = kind, rows, n, _act(x), p0, p1
     a.x_stride, a.gate_stride, a.out_stride = x.stride(0), (0 if gate is None else gate.stride(0)), out.stride(0)
+    if gate_rows is not None:
+        a.gate_rows, a.gate_row_count = _p(gate_rows), gate.shape[0]
     _C.check(_C.load().hymeta_activation(C.byref(a), _stream(x)), "hymeta_activation")
     return out
 
@@ -2069,6 +2138,20 @@ def silu_mul(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tenso
     bf16-only form of the quantised linears' path)."""
     _require(x.shape[1] % 2 == 0, "x must hold the gate and the up columns")
     return _activation(_C.ACT_SILU_MUL, x, x.shape[1] // 2, 0.0, 0.0, out=out)
+
+
+def gelu_mul(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``x [rows, 2 n]`` (gate columns, then up columns) -> ``gelu(gate) up``, gelu in its tanh form, bf16 or fp32."""
+    _require(x.shape[1] % 2 == 0, "x must hold the gate and the up columns")
+    return _activation(_C.ACT_GELU_MUL, x, x.shape[1] // 2, 0.0, 0.0, out=out)
+
+
+def gelu_mul_rows(x: torch.Tensor, table: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
+    """``gelu(x) * table[rows]``: ``x [T, n]``, ``table [entries, n]`` (a view with any row stride, x's type), ``rows`` int64
+    ``[T]``; gelu in its tanh form."""
+    _require(table.dim() == 2 and table.shape[1] == x.shape[1] and table.stride(1) == 1 and table.dtype == x.dtype, "table must be row-contiguous [entries, n] of x's type")
+    _require(rows.dtype == torch.int64 and rows.is_contiguous() and rows.numel() == x.shape[0], "rows must be int64 [T]")
+    return _activation(_C.ACT_GELU_ROWS, x, x.shape[1], 0.0, 0.0, gate=table, gate_rows=rows)
 
 
 def relu_squared(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -2340,4 +2423,58 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.T
         ws = _workspace(q.device, nbytes, "decay_scan")
         a.workspace, a.workspace_bytes = _p(ws), ws.numel()
     _C.check(lib.hymeta_decay_scan(C.byref(a), _stream(q)), "hymeta_decay_scan")
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Gated delta rule.
+# ---------------------------------------------------------------------------
+def delta_rule_step_supported(head_dim: int, v_dim: int) -> bool:
+    """Whether single rows run the step kernel (and with it the output norm in the same launch)."""
+    return v_dim % 4 == 0 and v_dim <= 1024 and 256 % (v_dim // 4) == 0 and head_dim <= 256 and head_dim * (v_dim // 4) <= 4096
+
+
+def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, beta_logit: torch.Tensor, log2_decay: torch.Tensor, state: torch.Tensor,
+               query_start_loc: torch.Tensor, context_lens: torch.Tensor, slot_idx: torch.Tensor, max_query_len: int, q_scale: float,
+               unit_eps: float, norm_weight: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+               norm_eps: float = 0.0) -> torch.Tensor:
+    """``S <- 2^log2_decay S; u = sigmoid(beta_logit) (v - S^T k'); S <- S + k' u^T; o = S^T q'`` over a step's rows, with
+    ``k' = k / sqrt(sum(k^2) + unit_eps)`` and ``q' = q_scale q / sqrt(sum(q^2) + unit_eps)``: ``q, k [T, Hqk, D]``, ``v [T, H,
+    Dv]``, ``beta_logit [T, H]`` (views with any row stride; head ``h`` reads query / key head ``h // (H / Hqk)``), ``log2_decay``
+    fp32 ``[T, H]``, ``state`` fp32 ``[slots, H, D, Dv]`` read where ``context_lens > 0`` and written.  Returns fp32 ``[T, H Dv]``;
+    with ``norm_weight [Dv]`` (a step of single rows, ``delta_rule_step_supported``) ``rmsnorm(o) * norm_weight * silu(gate)``
+    per head in the activations' type."""
+    _dev(q, k, v, beta_logit, log2_decay, state, query_start_loc, context_lens, slot_idx, norm_weight, gate)
+    _require(q.dim() == 3 and k.shape == q.shape and v.dim() == 3 and q.dtype == k.dtype == v.dtype == beta_logit.dtype and q.dtype in _DT,
+             "q, k [T, Hqk, D], v [T, H, Dv] and beta_logit [T, H] of one type")
+    T, Hqk, D = q.shape
+    H, Dv = v.shape[1], v.shape[2]
+    for t_, n_ in ((q, D), (k, D), (v, Dv)):
+        _require(t_.shape[0] == T and t_.stride(2) == 1 and t_.stride(1) == n_, "heads must be contiguous in a row")
+    _require(H % Hqk == 0, "the heads must split over the query / key heads")
+    _require(beta_logit.shape == (T, H) and beta_logit.stride(1) == 1, "beta_logit must be row-contiguous [T, H]")
+    _require(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 4 and state.shape[1:] == (H, D, Dv),
+             "state must be contiguous fp32 [slots, H, D, Dv]")
+    _f32vec(log2_decay, T * H, "log2_decay")
+    _f32vec(norm_weight, Dv, "norm_weight")
+    S = query_start_loc.numel() - 1
+    _i32vec(query_start_loc, S + 1, "query_start_loc")
+    _i32vec(context_lens, S, "context_lens")
+    _i32vec(slot_idx, S, "slot_idx")
+    out = torch.empty(T, H * Dv, dtype=torch.float32 if norm_weight is None else q.dtype, device=q.device)
+    a = _C.DeltaRuleArgs()
+    a.q, a.k, a.v, a.beta_logit, a.log2_decay, a.state, a.out = _p(q), _p(k), _p(v), _p(beta_logit), _p(log2_decay), _p(state), _p(out)
+    a.query_start_loc, a.context_lens, a.slot_idx = _p(query_start_loc), _p(context_lens), _p(slot_idx)
+    a.num_tokens, a.num_seqs, a.num_heads, a.num_qk_heads, a.head_dim, a.v_dim = T, S, H, Hqk, D, Dv
+    a.act_dtype, a.max_query_len, a.q_scale, a.unit_eps, a.norm_eps = _act(q), max_query_len, float(q_scale), float(unit_eps), float(norm_eps)
+    a.q_stride_t, a.k_stride_t, a.v_stride_t, a.beta_stride_t = q.stride(0), k.stride(0), v.stride(0), beta_logit.stride(0)
+    if norm_weight is not None:
+        _require(gate is not None and gate.shape == (T, H * Dv) and gate.stride(1) == 1 and gate.dtype == q.dtype, "gate must be row-contiguous [T, H Dv] of q's type")
+        a.norm_weight, a.gate, a.gate_stride_t = _p(norm_weight), _p(gate), gate.stride(0)
+    lib = _C.load()
+    nbytes = int(lib.hymeta_delta_rule_workspace_bytes(T, S, H, Hqk, D, Dv, a.act_dtype, max_query_len))
+    if nbytes:
+        ws = _workspace(q.device, nbytes, "delta_rule")
+        a.workspace, a.workspace_bytes = _p(ws), ws.numel()
+    _C.check(lib.hymeta_delta_rule(C.byref(a), _stream(q)), "hymeta_delta_rule")
     return out

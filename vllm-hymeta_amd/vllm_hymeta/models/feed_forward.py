@@ -6,6 +6,7 @@
 ``SigmoidRoutedMoE``  experts of the second form chosen by the largest ``sigmoid`` router scores, weighing their scores
                     over the chosen's sum times a constant, beside an optional shared expert that every token runs
 ``SiluGluMLP``      ``W_down (silu(W_gate h + b_gate) (W_up h + b_up)) + b_down``, bf16 or fp32
+``GeluGluMLP``      ``W_down (gelu(W_gate h) (W_up h))``, gelu in its tanh form, bf16 or fp32
 ``Relu2RoutedMoE``  experts ``W_down max(W_up h, 0)^2`` chosen by the largest router logits ``W_r h + b_r``, weighing the
                     softmax over the chosen logits alone
 ``GroupedSoftmaxMoE``  silu-gated experts weighed by the softmax over ALL router outputs (not renormalised), chosen by
@@ -76,6 +77,16 @@ class SiluGluMLP(torch.nn.Module):
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         return self.down_proj(hip_ops.silu_mul(self.gate_up_proj(h)))
+
+
+class GeluGluMLP(torch.nn.Module):
+    def __init__(self, gate_up_proj: HymetaLinear, down_proj: HymetaLinear):
+        """``gate_up_proj``: rows = gate, then up."""
+        super().__init__()
+        self.gate_up_proj, self.down_proj = gate_up_proj, down_proj
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return self.down_proj(hip_ops.gelu_mul(self.gate_up_proj(h)))
 
 
 class Relu2RoutedMoE(torch.nn.Module):

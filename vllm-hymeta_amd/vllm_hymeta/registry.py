@@ -36,6 +36,11 @@ def _dapuzen_config(model_dir: str):
     return DapuzenConfig.from_pretrained(model_dir)
 
 
+def _nilevik_config(model_dir: str):
+    from .models.configuration_nilevik import NilevikConfig
+    return NilevikConfig.from_pretrained(model_dir)
+
+
 def _gla_swa_config(model_dir: str):
     from .model_for_7B.configuration_gla_swa import GLAswaConfig
     with open(os.path.join(model_dir, "config.json")) as f:
@@ -52,6 +57,8 @@ register("Lidizen", "vllm_hymeta.models.modeling_lidizen:LidizenForCausalLM", _l
 register("LidizenForCausalLM", "vllm_hymeta.models.modeling_lidizen:LidizenForCausalLM", _lidizen_config)
 register("Dapuzen", "vllm_hymeta.models.modeling_dapuzen:DapuzenForCausalLM", _dapuzen_config)
 register("DapuzenForCausalLM", "vllm_hymeta.models.modeling_dapuzen:DapuzenForCausalLM", _dapuzen_config)
+register("Nilevik", "vllm_hymeta.models.modeling_nilevik:NilevikForCausalLM", _nilevik_config)
+register("NilevikForCausalLM", "vllm_hymeta.models.modeling_nilevik:NilevikForCausalLM", _nilevik_config)
 register("GLAswaForCausalLM", "vllm_hymeta.model_for_7B.modeling_gla_swa:GLAswaForCausalLM", _gla_swa_config)
 
 
@@ -87,6 +94,8 @@ _KERNEL_SOURCES = {
                            "dense_gemm", "stream_gemm", "tall_gemm"),
     "DapuzenForCausalLM": ("api_misc", "norm_conv", "parallel_ops", "decay_scan", "lightning", "sink_attn", "gated_ops", "moe_sigmoid",
                            "moe_table", "moe", "glue", "dense_gemm", "stream_gemm", "tall_gemm"),
+    "NilevikForCausalLM": ("api_misc", "norm_conv", "parallel_ops", "lightning", "sink_attn", "delta_rule", "gated_ops", "glue",
+                           "dense_gemm", "stream_gemm", "tall_gemm"),
 }
 
 
