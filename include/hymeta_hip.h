@@ -715,8 +715,8 @@ int hymeta_bf16_gemm_takes(int32_t M, int32_t K, int32_t N, int32_t form);
 int hymeta_bf16_gemm_f32out(const hymeta_bf16_gemm_args* args, hymeta_stream_t stream);
 
 /* Greedy sampling of a decode step: out[m] = index of the largest of logits[m, 0 .. N) (fp32 rows stride_m elements
- * apart; the lowest index among equals), in launches that a captured decode step can hold.  N and stride_m
- * multiples of 4.  workspace (hymeta_argmax_rows_workspace_bytes(M) bytes, or NULL) lets a wide row be scanned by 32
+ * apart; the lowest index among equals), in launches that a captured decode step can hold.  Rows in
+ * whole fours (N, stride_m, address) are read 16 bytes at a time.  workspace (hymeta_argmax_rows_workspace_bytes(M) bytes, or NULL) lets a wide row be scanned by 32
  * workgroups with a second small launch picking among them; without it one workgroup scans a row.
  * Stands in for the argmax of vLLM's sampler on greedy requests (the reference hands its logits to that sampler:
  * vllm_hymeta/model_for_7B/modeling_gla_swa.py:579-590). */

@@ -488,18 +488,26 @@ namespace hymeta {
 // Greedy sampling: index of the largest logit of each row (the lowest index among equals).  A workgroup scans one of
 // ``segs`` column segments of a row, 4 columns per thread at a time, and merges its 256 candidates through LDS; with
 // more than one segment the candidates (value, index) go to ``part`` [M][segs] and a second launch picks among them.
+// Fours: rows, their stride and their start in whole fours (16-byte loads); else column by column.
+template <bool Fours>
 __global__ __launch_bounds__(256) void argmax_rows_kernel(const float* logits, int64_t stride, int n, int segs, float* part_val,
                                                           int* part_idx, int64_t* out) {
   __shared__ float s_val[256];
   __shared__ int s_idx[256];
   const int m = blockIdx.x / segs, seg = blockIdx.x % segs;
   const float* row = logits + static_cast<int64_t>(m) * stride;
-  const int per = ((n / 4 + segs - 1) / segs) * 4;            // columns per segment, a multiple of 4
+  const int per = (((n + 3) / 4 + segs - 1) / segs) * 4;            // columns per segment, a multiple of 4
   const int lo = seg * per, hi = min(n, lo + per);
   float best = -INFINITY;
   int best_i = 0x7fffffff;
   for (int c = lo + 4 * threadIdx.x; c < hi; c += 1024) {
-    const f32x4 v = *reinterpret_cast<const f32x4*>(row + c);
+    f32x4 v;
+    if (Fours) {
+      v = *reinterpret_cast<const f32x4*>(row + c);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = c + e < hi ? row[c + e] : -INFINITY;
+    }
 #pragma unroll
     for (int e = 0; e < 4; ++e)
       if (v[e] > best) best = v[e], best_i = c + e;       // ascending columns: the first of equals stays
@@ -543,14 +551,16 @@ extern "C" int hymeta_argmax_rows(const float* logits, int64_t stride_m, int32_t
   if (M < 0 || N <= 0) return HYMETA_ERR_INVALID_ARG;
   if (M == 0) return HYMETA_OK;
   if (!logits || !out) return HYMETA_ERR_INVALID_ARG;
-  if (N % 4 != 0 || stride_m % 4 != 0 || reinterpret_cast<uintptr_t>(logits) % 16 != 0) return HYMETA_ERR_UNSUPPORTED;
+  if (stride_m < N) return HYMETA_ERR_INVALID_ARG;
+  const bool fours = N % 4 == 0 && stride_m % 4 == 0 && reinterpret_cast<uintptr_t>(logits) % 16 == 0;
   // few rows of a wide vocabulary: 32 workgroups per row, so that the whole chip reads
   const int segs = workspace != nullptr && workspace_bytes >= hymeta_argmax_rows_workspace_bytes(M) && N >= 32 * 1024 && M <= 1024 &&
                            reinterpret_cast<uintptr_t>(workspace) % 4 == 0 ? 32 : 1;
   float* part_val = static_cast<float*>(workspace);
   int* part_idx = reinterpret_cast<int*>(part_val + static_cast<size_t>(M) * 32);
   hipStream_t s = hymeta::begin_launches(stream);
-  hipLaunchKernelGGL(hymeta::argmax_rows_kernel, dim3(M * segs), dim3(256), 0, s, logits, stride_m, N, segs, part_val, part_idx, out);
+  if (fours) hipLaunchKernelGGL(hymeta::argmax_rows_kernel<true>, dim3(M * segs), dim3(256), 0, s, logits, stride_m, N, segs, part_val, part_idx, out);
+  else hipLaunchKernelGGL(hymeta::argmax_rows_kernel<false>, dim3(M * segs), dim3(256), 0, s, logits, stride_m, N, segs, part_val, part_idx, out);
   if (segs > 1) {
     if (hipGetLastError() != hipSuccess) return HYMETA_ERR_LAUNCH;
     hipLaunchKernelGGL(hymeta::argmax_pick_kernel, dim3(M), dim3(64), 0, s, part_val, part_idx, segs, out);
