@@ -5,6 +5,8 @@
 // whose state only adds what a token brings.
 #include "act_types.h"
 
+#include <type_traits>
+
 namespace hymeta {
 
 namespace {
@@ -191,11 +193,19 @@ __global__ __launch_bounds__(256) void delta_rule_step_kernel(hymeta_delta_rule_
 // query_start_loc[s] / 64 + s + c, at most num_tokens / 64 + num_seqs of them.
 // ------------------------------------------------------------------------------------------------
 typedef float f32x4v __attribute__((ext_vector_type(4)));
-constexpr int kChunk = HYMETA_DELTA_CHUNK, kSliceV = 32;
+constexpr int kChunk = HYMETA_DELTA_CHUNK;
+// Workgroups (with slices of 32 value columns) up to which the second launch runs slices of 16: measured for one prompt of 8192
+// with 28 heads of 128 x 128 (112 workgroups) 357 against 405 us, with 64 heads (256) 706 against 566 us.
+constexpr int kFewGroups = 128;
 constexpr int kChunkMinRows = 8;            // shorter portions go token by token
 constexpr int kMat = kChunk * kChunk;
-// a chunk's and head's place in the workspace: T hi, T lo, P hi, P lo (bf16, row i's entries j consecutive), then per row
-// beta, beta 2^(c_i) / |k|, q_scale 2^(c_i) / |q|, 2^(c - c_j) / |k|, then 2^c
+// Where the second launch reads 64 x 64 matrices (or the chunk's keys) as matrix operands, they lie in the operand's own
+// order: per 16 rows and 32 columns the 64 lanes' 8 elements one after the other, so that a wave's load is 1 KB in a row.
+__device__ __forceinline__ int operand_at(int row, int col, int cols) {       // (col in whole fours)
+  return ((row >> 4) * (cols >> 5) + (col >> 5)) * 512 + (((col >> 3) & 3) * 16 + (row & 15)) * 8 + (col & 7);
+}
+// a chunk's and head's place in the workspace: T hi, T lo, P hi, P lo (bf16, operand order), then per row beta,
+// beta 2^(c_i) / |k|, q_scale 2^(c_i) / |q|, 2^(c - c_j) / |k|, then 2^c
 struct ChunkPlace {
   uint16_t t[2][kMat], p[2][kMat];
   float beta[kChunk], rhs[kChunk], read[kChunk], write[kChunk];
@@ -215,8 +225,9 @@ __device__ __forceinline__ void split4(const float* v, u32x2& hi, u32x2& lo) {
   }
 }
 
-// Workspace: the chunks' places ([chunk][head]), then per chunk and query / key head the chunk's keys transposed, [D][64] bf16.
-__host__ __device__ inline size_t transposed_at(int64_t chunks, int heads) { return static_cast<size_t>(chunks) * heads * sizeof(ChunkPlace); }
+// Workspace: the chunks' places ([chunk][head]), then per chunk and query / key head the chunk's keys [64][D], queries [64][D]
+// and transposed keys [D][64], bf16 in operand order.
+__host__ __device__ inline size_t rows_at(int64_t chunks, int heads) { return static_cast<size_t>(chunks) * heads * sizeof(ChunkPlace); }
 
 // grid = (chunk numbers, heads), 4 waves with 16 rows of the chunk each.
 template <int D>
@@ -286,7 +297,6 @@ __global__ __launch_bounds__(256) void delta_chunk_solve_kernel(hymeta_delta_rul
   const float ch = s_hi[i], cl = s_lo[i], bk = s_beta[i] * s_ik[i], iq = s_iq[i];
 #pragma unroll
   for (int jb = 0; jb < 4; ++jb) {
-    if (jb > (wave | 1)) break;
     float av[4] = {0.f, 0.f, 0.f, 0.f}, pv[4] = {0.f, 0.f, 0.f, 0.f};
     if (jb <= wave) {
       f32x4v xk = f32x4v{0.f, 0.f, 0.f, 0.f}, xq = xk;
@@ -306,11 +316,11 @@ __global__ __launch_bounds__(256) void delta_chunk_solve_kernel(hymeta_delta_rul
       }
       *reinterpret_cast<f32x4v*>(&sA[i * PF + 16 * jb + 4 * g4]) = f32x4v{av[0], av[1], av[2], av[3]};
     }
-    // (the block behind the diagonal is stored as zeros where the products over 32 rows reach it)
+    // (the blocks behind the diagonal are stored as zeros: every wave multiplies all 64 rows)
     u32x2 hi, lo;
     split4(pv, hi, lo);
-    *reinterpret_cast<u32x2*>(&place->p[0][i * kChunk + 16 * jb + 4 * g4]) = hi;
-    *reinterpret_cast<u32x2*>(&place->p[1][i * kChunk + 16 * jb + 4 * g4]) = lo;
+    *reinterpret_cast<u32x2*>(&place->p[0][operand_at(i, 16 * jb + 4 * g4, kChunk)]) = hi;
+    *reinterpret_cast<u32x2*>(&place->p[1][operand_at(i, 16 * jb + 4 * g4, kChunk)]) = lo;
   }
   __syncthreads();
   // T: the diagonal blocks by forward substitution, a column per lane (the four groups of lanes do the same)
@@ -352,32 +362,36 @@ __global__ __launch_bounds__(256) void delta_chunk_solve_kernel(hymeta_delta_rul
   }
   {
     const int row = tid >> 2, jb = tid & 3, rb = row >> 4;
-    if (jb <= (rb | 1)) {
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        float v[4] = {0.f, 0.f, 0.f, 0.f};
-        if (jb <= rb) {
-          const f32x4v tv = *reinterpret_cast<const f32x4v*>(&sT[row * PF + 16 * jb + 4 * u]);
+    for (int u = 0; u < 4; ++u) {
+      float v[4] = {0.f, 0.f, 0.f, 0.f};
+      if (jb <= rb) {
+        const f32x4v tv = *reinterpret_cast<const f32x4v*>(&sT[row * PF + 16 * jb + 4 * u]);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = tv[e];
-        }
-        u32x2 hi, lo;
-        split4(v, hi, lo);
-        *reinterpret_cast<u32x2*>(&place->t[0][row * kChunk + 16 * jb + 4 * u]) = hi;
-        *reinterpret_cast<u32x2*>(&place->t[1][row * kChunk + 16 * jb + 4 * u]) = lo;
+        for (int e = 0; e < 4; ++e) v[e] = tv[e];
       }
+      u32x2 hi, lo;
+      split4(v, hi, lo);
+      *reinterpret_cast<u32x2*>(&place->t[0][operand_at(row, 16 * jb + 4 * u, kChunk)]) = hi;
+      *reinterpret_cast<u32x2*>(&place->t[1][operand_at(row, 16 * jb + 4 * u, kChunk)]) = lo;
     }
   }
   if (h % group == 0) {
-    uint16_t* kt = reinterpret_cast<uint16_t*>(static_cast<char*>(a.workspace) + transposed_at(chunks, H)) +
-                   (static_cast<int64_t>(number) * a.num_qk_heads + g) * D * kChunk;
+    uint16_t* kr = reinterpret_cast<uint16_t*>(static_cast<char*>(a.workspace) + rows_at(chunks, H)) +
+                   (static_cast<int64_t>(number) * a.num_qk_heads + g) * 3 * D * kChunk;
+    uint16_t *qr = kr + D * kChunk, *kt = qr + D * kChunk;
+#pragma unroll
+    for (int sd = 0; sd < D / 32; ++sd) {
+      st16(kr + operand_at(i, 32 * sd + 8 * g4, D), kf[sd]);
+      st16(qr + operand_at(i, 32 * sd + 8 * g4, D), qf[sd]);
+    }
     for (int idx = tid; idx < D * (kChunk / 8); idx += 256) {
       const int d = idx % D, tc = idx / D;
       u32x4 w;
 #pragma unroll
       for (int u = 0; u < 4; ++u)
         w[u] = static_cast<uint32_t>(sk[(8 * tc + 2 * u) * PK + d]) | (static_cast<uint32_t>(sk[(8 * tc + 2 * u + 1) * PK + d]) << 16);
-      st16(kt + d * kChunk + 8 * tc, w);
+      st16(kt + operand_at(d, 8 * tc, kChunk), w);
     }
   }
   if (wave == 0) {
@@ -391,34 +405,36 @@ __global__ __launch_bounds__(256) void delta_chunk_solve_kernel(hymeta_delta_rul
   }
 }
 
-// grid = (heads, sequences, value columns in slices of 32), 4 waves.  The state slice stays fp32 in registers in blocks of
+// grid = (heads, sequences, value columns in slices of 16 CB), 4 waves.  The state slice stays fp32 in registers in blocks of
 // 16 x 16 dealt over the waves (a lane holds 4 consecutive rows d of one column); its bf16 parts, the right-hand side and
 // U pass through LDS with the reduced index consecutive; everything a chunk brings comes from memory in the matrix
-// operands' own layout, loaded a chunk ahead.
-template <int D>
+// operands' own layout, loaded two chunks ahead (the loads of two chunks are in flight, each in registers of its own).  Rows past the portion read its last row (beta, and with it what they would
+// write, is 0 there), and the last chunk fetches itself once more, so that no load stands under a condition.
+template <int D, int CB>
 __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(hymeta_delta_rule_args a, int64_t chunks) {
-  constexpr int PK = D + 8, PT = kChunk + 8, NBW = D / 32;
-  __shared__ __attribute__((aligned(16))) uint16_t sst[2][kSliceV * PK];                                             // state, [c][d]
-  __shared__ __attribute__((aligned(16))) uint16_t srt[2][kSliceV * PT], su[2][kSliceV * PT], sw[2][kSliceV * PT];   // [c][row]
+  constexpr int SV = 16 * CB, PK = D + 8, PT = kChunk + 8, NBW = (D / 16) * CB / 4;
+  static_assert((D / 16) * CB % 4 == 0, "the state's blocks deal evenly over the waves");
+  __shared__ __attribute__((aligned(16))) uint16_t sst[2][SV * PK];                                      // state, [c][d]
+  __shared__ __attribute__((aligned(16))) uint16_t srt[2][SV * PT], su[2][SV * PT], sw[2][SV * PT];      // [c][row]
   const int h = blockIdx.x, s = blockIdx.y, vs = blockIdx.z;
   const int r0 = a.query_start_loc[s], rows = a.query_start_loc[s + 1] - r0;
   if (rows < kChunkMinRows) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n = lane & 15, g4 = lane >> 4;
   const int H = a.num_heads, G = a.num_qk_heads, Dv = a.v_dim, g = h / (H / G);
   const int slot = a.slot_idx[s];
-  float* st = slot >= 0 ? a.state + ((static_cast<int64_t>(slot) * H + h) * D) * Dv + vs * kSliceV : nullptr;
+  float* st = slot >= 0 ? a.state + ((static_cast<int64_t>(slot) * H + h) * D) * Dv + vs * SV : nullptr;
   const bool carry = st != nullptr && a.context_lens[s] > 0;
   f32x4v S[NBW];
 #pragma unroll
   for (int ib = 0; ib < NBW; ++ib) {
-    const int b = wave + 4 * ib, cb = b & 1, db = b >> 1;
+    const int b = wave + 4 * ib, cb = b % CB, db = b / CB;
 #pragma unroll
     for (int r = 0; r < 4; ++r) S[ib][r] = carry ? st[static_cast<int64_t>(16 * db + 4 * g4 + r) * Dv + 16 * cb + n] : 0.f;
   }
   auto state_to_lds = [&]() {
 #pragma unroll
     for (int ib = 0; ib < NBW; ++ib) {
-      const int b = wave + 4 * ib, cb = b & 1, db = b >> 1;
+      const int b = wave + 4 * ib, cb = b % CB, db = b / CB;
       const float v[4] = {S[ib][0], S[ib][1], S[ib][2], S[ib][3]};
       u32x2 hi, lo;
       split4(v, hi, lo);
@@ -427,161 +443,174 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(hymeta_delta_rule
     }
   };
   state_to_lds();
-  const uint16_t* qp = static_cast<const uint16_t*>(a.q) + static_cast<int64_t>(g) * D + 8 * g4;
-  const uint16_t* kp = static_cast<const uint16_t*>(a.k) + static_cast<int64_t>(g) * D + 8 * g4;
-  const uint16_t* vp = static_cast<const uint16_t*>(a.v) + static_cast<int64_t>(h) * Dv + vs * kSliceV + n;
+  const uint16_t* vp = static_cast<const uint16_t*>(a.v) + static_cast<int64_t>(h) * Dv + vs * SV + n;
   const int64_t first = r0 / kChunk + s;
   const ChunkPlace* places = static_cast<const ChunkPlace*>(a.workspace) + first * H + h;
-  const uint16_t* transposed = reinterpret_cast<const uint16_t*>(static_cast<const char*>(a.workspace) + transposed_at(chunks, H)) +
-                               (first * G + g) * D * kChunk;
-  const int i = 16 * wave + n;              // the row of this lane's operand fragments
+  const uint16_t* packed = reinterpret_cast<const uint16_t*>(static_cast<const char*>(a.workspace) + rows_at(chunks, H)) +
+                           (first * G + g) * 3 * D * kChunk + 8 * lane;          // keys, queries, transposed keys of the chunks
   const int iq = 16 * wave + 4 * g4;        // the first of the four rows of this lane's results
-  const int kks = wave < 2 ? 1 : 2;         // blocks of 32 rows up to the wave's own
-  u32x4 kf[D / 32], qf[D / 32], tf[2][2], pf[2][2], wf[NBW][2];
-  uint16_t vv[2][4];
-  f32x4v beta, rhs, read, write;
-  float total;
-  auto fetch_rows = [&](int c) {
-    const int nrow = min(kChunk, rows - c * kChunk);
-    const int64_t t0 = r0 + static_cast<int64_t>(c) * kChunk;
-#pragma unroll
-    for (int sd = 0; sd < D / 32; ++sd) {
-      kf[sd] = qf[sd] = u32x4{0u, 0u, 0u, 0u};
-      if (i < nrow) kf[sd] = ld16g(kp + (t0 + i) * a.k_stride_t + 32 * sd), qf[sd] = ld16g(qp + (t0 + i) * a.q_stride_t + 32 * sd);
-    }
-#pragma unroll
-    for (int cb = 0; cb < 2; ++cb)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) vv[cb][r] = iq + r < nrow ? vp[(t0 + iq + r) * a.v_stride_t + 16 * cb] : static_cast<uint16_t>(0);
+  // what a chunk brings: row fragments of the keys, queries, T and P, the transposed keys of this wave's state blocks, values
+  struct Chunk {
+    u32x4 kf[D / 32], qf[D / 32], tf[2][2], pf[2][2], wf[NBW][2];
+    uint16_t vv[CB][4];
+    f32x4v beta, rhs, read, write;
+    float total;
   };
-  auto fetch_solved = [&](int c, bool t_part) {
+  auto fetch_rows = [&](Chunk& m, int c) {
+    const int last = rows - 1 - c * kChunk;
+    const int64_t t0 = r0 + static_cast<int64_t>(c) * kChunk;
+    const uint16_t* kr = packed + static_cast<int64_t>(c) * G * 3 * D * kChunk + wave * (D / 32) * 512;
+#pragma unroll
+    for (int sd = 0; sd < D / 32; ++sd) m.kf[sd] = ld16g(kr + 512 * sd), m.qf[sd] = ld16g(kr + D * kChunk + 512 * sd);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const uint16_t* vr = vp + (t0 + min(iq + r, last)) * a.v_stride_t;
+#pragma unroll
+      for (int cb = 0; cb < CB; ++cb) m.vv[cb][r] = vr[16 * cb];
+    }
+  };
+  auto fetch_t = [&](Chunk& m, int c) {
     const ChunkPlace* p = places + static_cast<int64_t>(c) * H;
 #pragma unroll
     for (int part = 0; part < 2; ++part)
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk)
-        if (kk < kks) {
-          if (t_part) tf[part][kk] = ld16g(&p->t[part][i * kChunk + 32 * kk + 8 * g4]);
-          else pf[part][kk] = ld16g(&p->p[part][i * kChunk + 32 * kk + 8 * g4]);
-        }
-    if (t_part) {
-      beta = *reinterpret_cast<const f32x4v*>(&p->beta[iq]);
-      rhs = *reinterpret_cast<const f32x4v*>(&p->rhs[iq]);
-      read = *reinterpret_cast<const f32x4v*>(&p->read[iq]);
-      write = *reinterpret_cast<const f32x4v*>(&p->write[iq]);
-      total = p->total;
-    }
+      for (int kk = 0; kk < 2; ++kk) m.tf[part][kk] = ld16g(&p->t[part][(2 * wave + kk) * 512 + 8 * lane]);
+    m.beta = *reinterpret_cast<const f32x4v*>(&p->beta[iq]);
+    m.rhs = *reinterpret_cast<const f32x4v*>(&p->rhs[iq]);
+    m.read = *reinterpret_cast<const f32x4v*>(&p->read[iq]);
+    m.write = *reinterpret_cast<const f32x4v*>(&p->write[iq]);
   };
-  auto fetch_transposed = [&](int c) {
-    const uint16_t* kt = transposed + static_cast<int64_t>(c) * G * D * kChunk;
+  auto fetch_p = [&](Chunk& m, int c) {
+    const ChunkPlace* p = places + static_cast<int64_t>(c) * H;
+#pragma unroll
+    for (int part = 0; part < 2; ++part)
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) m.pf[part][kk] = ld16g(&p->p[part][(2 * wave + kk) * 512 + 8 * lane]);
+  };
+  auto fetch_transposed = [&](Chunk& m, int c) {
+    const uint16_t* kt = packed + (static_cast<int64_t>(c) * G * 3 + 2) * D * kChunk;
+    m.total = places[static_cast<int64_t>(c) * H].total;
 #pragma unroll
     for (int ib = 0; ib < NBW; ++ib) {
-      const int db = (wave + 4 * ib) >> 1;
+      const int db = (wave + 4 * ib) / CB;
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk) wf[ib][kk] = ld16g(kt + (16 * db + n) * kChunk + 32 * kk + 8 * g4);
+      for (int kk = 0; kk < 2; ++kk) m.wf[ib][kk] = ld16g(kt + (2 * db + kk) * 512);
     }
   };
-  fetch_rows(0);
-  fetch_solved(0, true);
-  fetch_solved(0, false);
-  fetch_transposed(0);
-  float* out = static_cast<float*>(a.out);
+  float* out = static_cast<float*>(a.out) + static_cast<int64_t>(r0) * H * Dv + static_cast<int64_t>(h) * Dv + vs * SV + n;
   const int num = (rows + kChunk - 1) / kChunk;
-  for (int c = 0; c < num; ++c) {
-    const bool more = c + 1 < num;
+  auto advance = [&](Chunk& m, int c, auto full) {         // full: a whole chunk (every row is the portion's)
+    const int next = min(c + 2, num - 1);
     __syncthreads();                        // the state's parts are in place
-    f32x4v x[2], y[2];
+    f32x4v x[CB], y[CB];
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) {
+    for (int cb = 0; cb < CB; ++cb) {
       x[cb] = y[cb] = f32x4v{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int sd = 0; sd < D / 32; ++sd) {
         const bf16x8 sh = frag(ld16(&sst[0][(16 * cb + n) * PK + 32 * sd + 8 * g4]));
         const bf16x8 sl = frag(ld16(&sst[1][(16 * cb + n) * PK + 32 * sd + 8 * g4]));
-        x[cb] = mfma16(frag(kf[sd]), sh, x[cb]);
-        y[cb] = mfma16(frag(qf[sd]), sh, y[cb]);
-        x[cb] = mfma16(frag(kf[sd]), sl, x[cb]);
-        y[cb] = mfma16(frag(qf[sd]), sl, y[cb]);
+        x[cb] = mfma16(frag(m.kf[sd]), sh, x[cb]);
+        y[cb] = mfma16(frag(m.qf[sd]), sh, y[cb]);
+        x[cb] = mfma16(frag(m.kf[sd]), sl, x[cb]);
+        y[cb] = mfma16(frag(m.qf[sd]), sl, y[cb]);
       }
     }
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) {
+    for (int cb = 0; cb < CB; ++cb) {
       float v[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        v[r] = beta[r] * bf2f(vv[cb][r]) - rhs[r] * x[cb][r];
-        y[cb][r] *= read[r];
+        v[r] = m.beta[r] * bf2f(m.vv[cb][r]) - m.rhs[r] * x[cb][r];
+        y[cb][r] *= m.read[r];
       }
       u32x2 hi, lo;
       split4(v, hi, lo);
       *reinterpret_cast<u32x2*>(&srt[0][(16 * cb + n) * PT + iq]) = hi;
       *reinterpret_cast<u32x2*>(&srt[1][(16 * cb + n) * PT + iq]) = lo;
     }
-    if (more) fetch_rows(c + 1);
-    const f32x4v wr = write;
-    const float tot = total;
+    fetch_rows(m, next);
     __syncthreads();
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) {
+    for (int cb = 0; cb < CB; ++cb) {
       f32x4v u = f32x4v{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk)
-        if (kk < kks) {
-          const bf16x8 rh = frag(ld16(&srt[0][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
-          const bf16x8 rl = frag(ld16(&srt[1][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
-          u = mfma16(frag(tf[0][kk]), rh, u);
-          u = mfma16(frag(tf[0][kk]), rl, u);
-          u = mfma16(frag(tf[1][kk]), rh, u);
-        }
+      for (int kk = 0; kk < 2; ++kk) {
+        const bf16x8 rh = frag(ld16(&srt[0][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
+        const bf16x8 rl = frag(ld16(&srt[1][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
+        u = mfma16(frag(m.tf[0][kk]), rh, u);
+        u = mfma16(frag(m.tf[0][kk]), rl, u);
+        u = mfma16(frag(m.tf[1][kk]), rh, u);
+      }
       float v[4] = {u[0], u[1], u[2], u[3]};
       u32x2 hi, lo;
       split4(v, hi, lo);
       *reinterpret_cast<u32x2*>(&su[0][(16 * cb + n) * PT + iq]) = hi;
       *reinterpret_cast<u32x2*>(&su[1][(16 * cb + n) * PT + iq]) = lo;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) v[r] *= wr[r];
+      for (int r = 0; r < 4; ++r) v[r] *= m.write[r];
       split4(v, hi, lo);
       *reinterpret_cast<u32x2*>(&sw[0][(16 * cb + n) * PT + iq]) = hi;
       *reinterpret_cast<u32x2*>(&sw[1][(16 * cb + n) * PT + iq]) = lo;
     }
-    if (more) fetch_solved(c + 1, true);
+    fetch_t(m, next);
     __syncthreads();
-    const int nrow = min(kChunk, rows - c * kChunk);
 #pragma unroll
     for (int ib = 0; ib < NBW; ++ib) {
-      const int cb = (wave + 4 * ib) & 1;
-      f32x4v acc = S[ib] * tot;
+      const int cb = (wave + 4 * ib) % CB;
+      f32x4v acc = S[ib] * m.total;
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
-        acc = mfma16(frag(wf[ib][kk]), frag(ld16(&sw[0][(16 * cb + n) * PT + 32 * kk + 8 * g4])), acc);
-        acc = mfma16(frag(wf[ib][kk]), frag(ld16(&sw[1][(16 * cb + n) * PT + 32 * kk + 8 * g4])), acc);
+        acc = mfma16(frag(m.wf[ib][kk]), frag(ld16(&sw[0][(16 * cb + n) * PT + 32 * kk + 8 * g4])), acc);
+        acc = mfma16(frag(m.wf[ib][kk]), frag(ld16(&sw[1][(16 * cb + n) * PT + 32 * kk + 8 * g4])), acc);
       }
       S[ib] = acc;
     }
-    if (more) fetch_transposed(c + 1);
+    fetch_transposed(m, next);
     state_to_lds();                         // (its last readers passed the barrier before)
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) {
+    for (int cb = 0; cb < CB; ++cb) {
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk)
-        if (kk < kks) {
-          const bf16x8 uh = frag(ld16(&su[0][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
-          const bf16x8 ul = frag(ld16(&su[1][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
-          y[cb] = mfma16(frag(pf[0][kk]), uh, y[cb]);
-          y[cb] = mfma16(frag(pf[0][kk]), ul, y[cb]);
-          y[cb] = mfma16(frag(pf[1][kk]), uh, y[cb]);
-        }
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (iq + r < nrow)
-          out[(r0 + static_cast<int64_t>(c) * kChunk + iq + r) * H * Dv + static_cast<int64_t>(h) * Dv + vs * kSliceV + 16 * cb + n] = y[cb][r];
+      for (int kk = 0; kk < 2; ++kk) {
+        const bf16x8 uh = frag(ld16(&su[0][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
+        const bf16x8 ul = frag(ld16(&su[1][(16 * cb + n) * PT + 32 * kk + 8 * g4]));
+        y[cb] = mfma16(frag(m.pf[0][kk]), uh, y[cb]);
+        y[cb] = mfma16(frag(m.pf[0][kk]), ul, y[cb]);
+        y[cb] = mfma16(frag(m.pf[1][kk]), uh, y[cb]);
+      }
     }
-    if (more) fetch_solved(c + 1, false);
+    fetch_p(m, next);
+    const int live = rows - c * kChunk - iq;            // rows of this lane's four that are the portion's
+    float* to = out + (static_cast<int64_t>(c) * kChunk + iq) * H * Dv;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (decltype(full)::value || r < live) {
+#pragma unroll
+        for (int cb = 0; cb < CB; ++cb) to[static_cast<int64_t>(r) * H * Dv + 16 * cb] = y[cb][r];
+      }
+  };
+  Chunk even, odd;
+  auto fetch = [&](Chunk& m, int c) {
+    fetch_rows(m, c);
+    fetch_t(m, c);
+    fetch_transposed(m, c);
+    fetch_p(m, c);
+  };
+  fetch(even, 0);
+  fetch(odd, min(1, num - 1));
+  // (the loop's body has no branch: loads under one, or a chunk that might not run, would make the waits in front of the
+  // matrix products wait for the loads of the chunks behind as well)
+  int c = 0;
+  for (; c + 2 < num; c += 2) {
+    advance(even, c, std::true_type{});
+    advance(odd, c + 1, std::true_type{});
   }
+  advance(even, c, std::false_type{});
+  if (c + 1 < num) advance(odd, c + 1, std::false_type{});
   if (st != nullptr) {
 #pragma unroll
     for (int ib = 0; ib < NBW; ++ib) {
-      const int b = wave + 4 * ib, cb = b & 1, db = b >> 1;
+      const int b = wave + 4 * ib, cb = b % CB, db = b / CB;
 #pragma unroll
       for (int r = 0; r < 4; ++r) st[static_cast<int64_t>(16 * db + 4 * g4 + r) * Dv + 16 * cb + n] = S[ib][r];
     }
@@ -589,7 +618,7 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(hymeta_delta_rule
 }
 
 inline bool chunk_dims(int head_dim, int v_dim, int act_dtype) {
-  return act_dtype == HYMETA_BF16 && head_dim >= 32 && head_dim <= 128 && head_dim % 32 == 0 && v_dim % kSliceV == 0 && v_dim / kSliceV <= 65535;
+  return act_dtype == HYMETA_BF16 && head_dim >= 32 && head_dim <= 128 && head_dim % 32 == 0 && v_dim % 32 == 0 && v_dim / 16 <= 65535;
 }
 inline bool chunk_shape(const hymeta_delta_rule_args& a) {
   auto aligned = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
@@ -616,7 +645,14 @@ void launch_rows(const hymeta_delta_rule_args& a, hipStream_t st, int min_rows, 
 template <int D>
 void launch_chunks(const hymeta_delta_rule_args& a, hipStream_t st, int64_t chunks) {
   hipLaunchKernelGGL(delta_chunk_solve_kernel<D>, dim3(static_cast<unsigned>(chunks), a.num_heads), dim3(256), 0, st, a, chunks);
-  hipLaunchKernelGGL(delta_chunk_scan_kernel<D>, dim3(a.num_heads, a.num_seqs, a.v_dim / kSliceV), dim3(256), 0, st, a, chunks);
+  // slices of 32 columns reread a chunk's matrices half as often; slices of 16 double the workgroups where they are few
+  if constexpr (D % 64 == 0) {
+    if (static_cast<int64_t>(a.num_heads) * a.num_seqs * (a.v_dim / 32) <= kFewGroups) {
+      hipLaunchKernelGGL((delta_chunk_scan_kernel<D, 1>), dim3(a.num_heads, a.num_seqs, a.v_dim / 16), dim3(256), 0, st, a, chunks);
+      return;
+    }
+  }
+  hipLaunchKernelGGL((delta_chunk_scan_kernel<D, 2>), dim3(a.num_heads, a.num_seqs, a.v_dim / 32), dim3(256), 0, st, a, chunks);
 }
 
 }  // namespace
@@ -629,7 +665,7 @@ extern "C" size_t hymeta_delta_rule_workspace_bytes(int32_t num_tokens, int32_t 
                                                     int32_t v_dim, int32_t act_dtype, int32_t max_query_len) {
   if (num_tokens <= 0 || num_seqs <= 0 || num_heads <= 0 || num_qk_heads <= 0 || max_query_len < kChunkMinRows || !chunk_dims(head_dim, v_dim, act_dtype)) return 0;
   const int64_t chunks = chunk_numbers(num_tokens, num_seqs);
-  return transposed_at(chunks, num_heads) + static_cast<size_t>(chunks) * num_qk_heads * head_dim * kChunk * 2;
+  return rows_at(chunks, num_heads) + static_cast<size_t>(chunks) * num_qk_heads * 3 * head_dim * kChunk * 2;
 }
 
 extern "C" int hymeta_delta_rule(const hymeta_delta_rule_args* args, hymeta_stream_t stream) {
