@@ -602,6 +602,72 @@ def test_long_decode_passes_every_window_and_keeps_its_states(dtype, name):
         assert rel_err(eng.run_batch([("x", toks[:201], [200])]), nilevik_ref(cfg, weights, toks[:201])[-1:]) < TOL[dtype]
 
 
+@pytest.mark.parametrize("name", ["default", "matrix_core_sizes"])
+def test_a_decode_step_replayed_from_a_graph(name):
+    """Three sequences of different lengths decode eight tokens: the step captured once and replayed, with eager work and
+    synchronisations between the replays, against the engine's eager steps."""
+    from vllm_hymeta.attention.meta_attention import MetaAttentionMetadata
+    from vllm_hymeta.models.attention import bind_kv_cache
+    cfg = nilevik_config(**MODELS[name])
+    weights = nilevik_random_weights(cfg, seed=3)
+    prompts, new, page, blocks = [_tokens(n, cfg["vocab"], n) for n in (90, 5, 64)], 8, 64, 2
+    fed = torch.tensor([_tokens(new, cfg["vocab"], 70 + s) for s in range(3)])
+    eng = build_engine(cfg, weights, torch.bfloat16, max_tokens=6 * page, block_size=page, max_num_seqs=3)
+    for s, p in enumerate(prompts):
+        eng.run_batch([(f"s{s}", p, [])])
+    model = eng.model
+    tables = torch.zeros(3, blocks, dtype=torch.int32)
+    for s in range(3):
+        r = eng.requests[f"s{s}"]
+        eng.pool.grow(r.blocks, len(prompts[s]) + new)
+        tables[s, :len(r.blocks)] = torch.tensor(r.blocks, dtype=torch.int32)
+    cache_before = {n: t.clone() for n, t in eng.kv_caches.items()}
+    states = model.model.state_cache._slot_tensors()
+    states_before = [t.clone() for t in states]
+    slots = [model.model.state_cache.slots.slot_of(eng.requests[f"s{s}"].state_key, 0) for s in range(3)]
+    want = [eng.run_batch([(f"s{s}", [int(fed[s, t])], [0]) for s in range(3)]) for t in range(new)]
+
+    def rewind():
+        for n, t in eng.kv_caches.items():
+            t.copy_(cache_before[n])
+            bind_kv_cache(eng.attn_layers[n], t)
+        for t, b in zip(states, states_before):
+            t.copy_(b)
+
+    lens = torch.tensor([len(p) for p in prompts])
+    ids, pos = torch.zeros(3, dtype=torch.int64, device=DEV), torch.zeros(3, dtype=torch.int64, device=DEV)
+    seq, ctx, sm = i32([0, 0, 0]), i32([0, 0, 0]), torch.zeros(3, dtype=torch.int64, device=DEV)
+    md = MetaAttentionMetadata(
+        num_prefills=0, num_prefill_tokens=0, num_decode_tokens=3, slot_mapping=sm, multi_modal_placeholder_index_maps=None,
+        enable_kv_scales_calculation=False, seq_lens=None, seq_lens_tensor=seq, max_prefill_seq_len=0, max_decode_seq_len=2 * page,
+        context_lens_tensor=ctx, block_tables=tables.to(DEV), use_cuda_graph=True, max_query_len=1, max_decode_query_len=1,
+        query_start_loc=i32([0, 1, 2, 3]), seq_start_loc=None)
+    cache, idx = model.get_seqlen_agnostic_capture_inputs(3)
+    idx.copy_(i32(slots))
+
+    def inputs(t):
+        p = lens + t
+        ids.copy_(fed[:, t]), pos.copy_(p), seq.copy_(p + 1), ctx.copy_(p)
+        sm.copy_(torch.tensor([int(tables[s, int(p[s]) // page]) * page + int(p[s]) % page for s in range(3)]))
+
+    with torch.inference_mode():
+        step = lambda: model.compute_logits(model(ids, pos, attn_metadata=md, seqlen_agnostic_capture_inputs=(cache, idx)))      # noqa: E731
+        inputs(0)
+        side, graph = torch.cuda.Stream(), torch.cuda.CUDAGraph()
+        with torch.cuda.stream(side):
+            step()
+            with torch.cuda.graph(graph, stream=side):
+                logits = step()
+        torch.cuda.synchronize()
+        rewind()
+        for t in range(new):
+            inputs(t)
+            graph.replay()
+            torch.cuda.synchronize()
+            assert rel_err(logits, want[t]) < 1e-3, t
+            torch.ones(1000, device=DEV).sum().item()
+
+
 def test_trace_runner_and_generate_command_lines(tmp_path):
     """A checkpoint folder (config.json + model.safetensors) served by the two programs under bin/: the trace replayer
     runs portions, single tokens and two requests side by side, gives pages back at a request's end and writes the logits
