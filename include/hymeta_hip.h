@@ -40,7 +40,10 @@
  *    version 8: hymeta_embed_rows_args ends with positions / pos_freqs / h_out, hymeta_norm_residual_args with h_out,
  *    hymeta_sink_attention_args with elem_gate / elem_gate_stride_t, hymeta_activation_args with gate_rows /
  *    gate_row_count; HYMETA_BIAS_LINEAR_DISTANCE, HYMETA_KV_SCALED_KEY, HYMETA_ACT_GELU_MUL / HYMETA_ACT_GELU_ROWS; the
- *    scaled-key cache and the delta rule at the end of this file).
+ *    scaled-key cache and the delta rule at the end of this file;
+ *    version 9: hymeta_sink_attention_args ends with chunk, hymeta_latent_kv_prep_args (q_rank may be 0) and
+ *    hymeta_latent_q_assemble_args with rot_half, hymeta_rotary_cache_args with interleaved / unit_rms / rot_mag /
+ *    unit_eps; hymeta_tanh_stream at the end of this file).
  *  - Every argument struct starts with `uint32_t struct_size`, which the caller
  *    sets to sizeof(the struct) of ITS declaration.  An entry point returns
  *    HYMETA_ERR_INVALID_ARG, before it reads any other field, when the value
@@ -58,7 +61,7 @@
 extern "C" {
 #endif
 
-#define HYMETA_ABI_VERSION 8
+#define HYMETA_ABI_VERSION 9
 
 typedef void* hymeta_stream_t;
 
@@ -1182,7 +1185,8 @@ int hymeta_qk_norm_cache(const hymeta_qk_norm_cache_args* args, hymeta_stream_t 
 
 /* Causal attention of a step's queries over their sequences' paged keys (the step's own keys are in
  * the cache already), with a distance bias and an optional sink:
- *   s_ij = scale * q_i . k_j - bias(i - j),   j <= i   (and i - j <= window_left when window_left >= 0)
+ *   s_ij = scale * q_i . k_j - bias(i - j),   j <= i   (and i - j <= window_left when window_left >= 0;
+ *   and i, j in the same run of `chunk` positions, counted from the sequence's first token, when chunk > 0)
  *   bias_mode HYMETA_BIAS_NONE: 0;  HYMETA_BIAS_LOG_DISTANCE: bias_a[h] * ln(1 + bias_b[h] * (i - j));
  *   HYMETA_BIAS_LINEAR_DISTANCE: bias_a[h] * (i - j)
  *   p_ij = exp(s_ij) / (sink + sum_j exp(s_ij)),  sink = exp(sink_logits[h]) (a key of that score, 0 without
@@ -1239,6 +1243,8 @@ typedef struct hymeta_sink_attention_args {
   const void* elem_gate;       /* act_dtype [num_tokens, num_heads * v_dim], row stride elem_gate_stride_t, or NULL: the
                                   output is multiplied element by element by sigmoid(elem_gate) */
   int64_t elem_gate_stride_t;
+  int32_t chunk;               /* > 0 (without window_left and keep_first): query i sees keys j <= i with
+                                  floor(j / chunk) == floor(i / chunk) */
 } hymeta_sink_attention_args;
 size_t hymeta_sink_attention_workspace_bytes(int32_t num_seqs, int32_t num_heads, int32_t num_kv_heads, int32_t v_dim,
                                              int32_t max_seq_len);
@@ -1338,8 +1344,9 @@ int hymeta_add_group_norm(const hymeta_add_group_norm_args* args, hymeta_stream_
  * by all heads (kv_rank + rot_dim columns from kv_col):
  *   query latent  <- RMS norm with q_norm_weight, in place
  *   cache row     <- (RMS norm of the key/value latent with kv_norm_weight, rotated key part)
- * kv_cache: act_dtype [num_blocks, block_size, kv_rank + rot_dim].  The rotation turns the pair (2i, 2i + 1), i <
- * rot_dims / 2 <= rot_dim / 2, by position * rot_freqs[i] (angles in double precision), cos and sin times rot_mag; the
+ * kv_cache: act_dtype [num_blocks, block_size, kv_rank + rot_dim].  The rotation turns the pair (2i, 2i + 1), or with
+ * rot_half (i, i + rot_dims / 2), i < rot_dims / 2 <= rot_dim / 2, by position * rot_freqs[i] (angles in double precision),
+ * cos and sin times rot_mag; q_rank 0: there is no query latent (q_norm_weight is not read); the
  * position of row t of sequence s is seq_lens[s] - (query_start_loc[s + 1] - t).  slot_mapping[t] < 0: no store. */
 typedef struct hymeta_latent_kv_prep_args {
   uint32_t struct_size;
@@ -1354,11 +1361,12 @@ typedef struct hymeta_latent_kv_prep_args {
   int32_t num_tokens, num_seqs, q_rank, kv_rank, rot_dim, rot_dims, q_col, kv_col, block_size, act_dtype;
   float eps, rot_mag;
   int64_t num_blocks, proj_stride_t;
+  int32_t rot_half;
 } hymeta_latent_kv_prep_args;
 int hymeta_latent_kv_prep(const hymeta_latent_kv_prep_args* args, hymeta_stream_t stream);
 
 /* The queries of a latent attention against the cached rows: out[t, h] = (q_abs[h, t] (kv_rank values: the unrotated
- * query part carried through the keys' up projection), rotated q[t, h, dim:] (rot_dim values)). */
+ * query part carried through the keys' up projection), rotated q[t, h, dim:] (rot_dim values, pairs as above)). */
 typedef struct hymeta_latent_q_assemble_args {
   uint32_t struct_size;
   const void* q;               /* act_dtype [num_tokens, num_heads, dim + rot_dim], row stride q_stride_t */
@@ -1370,6 +1378,7 @@ typedef struct hymeta_latent_q_assemble_args {
   int32_t num_tokens, num_seqs, num_heads, dim, rot_dim, rot_dims, kv_rank, act_dtype;
   float rot_mag;
   int64_t q_stride_t;
+  int32_t rot_half;
 } hymeta_latent_q_assemble_args;
 int hymeta_latent_q_assemble(const hymeta_latent_q_assemble_args* args, hymeta_stream_t stream);
 
@@ -1586,9 +1595,10 @@ typedef struct hymeta_stream_add_norm_args {
 int hymeta_stream_add_norm(const hymeta_stream_add_norm_args* args, hymeta_stream_t stream);
 
 /* Between a fused q | k | v (| ...) projection and an attention or a recurrence, per token, one launch, in place:
- *   of the first rot_dims dimensions of every query and key head, i and i + rot_dims / 2 turn together by
- *   position * rot_freqs[i] ("rotate half": (u, v) -> (u cos - v sin, v cos + u sin)); the rest pass; angles are reduced in
- *   double precision, the turn is fp32;
+ *   of the first rot_dims dimensions of every query and key head, i and i + rot_dims / 2 ("rotate half"), or with
+ *   interleaved 2 i and 2 i + 1, turn together by position * rot_freqs[i]: (u, v) -> (u cos - v sin, v cos + u sin), cos and
+ *   sin times rot_mag (0: 1); the rest pass; angles are reduced in double precision, the turn is fp32;
+ *   with unit_rms every query and key head is then divided by sqrt(mean over head_dim of its squares + unit_eps);
  *   keys are then multiplied by k_scale (0: by 1);
  *   with kv_cache: the cache row at slot_mapping[t] <- per key/value head the key followed by the value
  *   (HYMETA_KV_KEY_THEN_VALUE, as hymeta_sink_attention reads it).
@@ -1605,6 +1615,8 @@ typedef struct hymeta_rotary_cache_args {
   int32_t num_tokens, num_seqs, num_heads, num_kv_heads, head_dim, v_dim, rot_dims, block_size, act_dtype;
   float k_scale;
   int64_t num_blocks, qkv_stride_t;
+  int32_t interleaved, unit_rms;
+  float rot_mag, unit_eps;
 } hymeta_rotary_cache_args;
 int hymeta_rotary_cache(const hymeta_rotary_cache_args* args, hymeta_stream_t stream);
 
@@ -1729,6 +1741,30 @@ typedef struct hymeta_delta_rule_args {
 size_t hymeta_delta_rule_workspace_bytes(int32_t num_tokens, int32_t num_seqs, int32_t num_heads, int32_t num_qk_heads, int32_t head_dim,
                                          int32_t v_dim, int32_t act_dtype, int32_t max_query_len);
 int hymeta_delta_rule(const hymeta_delta_rule_args* args, hymeta_stream_t stream);
+
+/* Between two sublayers of a block whose norms squash instead of measuring, norm(v) = tanh(alpha v) weight + bias element by
+ * element, on the fp32 stream x, one launch:
+ *   with base:  x <- base (+ base2) (+ add)      (the stream starts anew from sums of products)
+ *   with y:     x <- x + tanh(y_alpha y) y_weight + y_bias
+ *   with h_out: h_out <- tanh(h_alpha x) h_weight + h_bias, or without h_weight x itself, rounded to act_dtype
+ * The stream is read unless base is given, and written unless neither base nor y is. */
+typedef struct hymeta_tanh_stream_args {
+  uint32_t struct_size;
+  float* x;                    /* [num_tokens, width], row stride x_stride_t */
+  const void* y;               /* act_dtype [num_tokens, width], row stride y_stride_t, or NULL */
+  const float* y_weight;       /* [width], and y_bias [width] (with y) */
+  const float* y_bias;
+  const float* base;           /* [num_tokens, width], row stride base_stride_t, or NULL */
+  const float* base2;          /* likewise (the same stride), or NULL */
+  const float* add;            /* [width] or NULL; read with base */
+  void* h_out;                 /* act_dtype [num_tokens, width] contiguous, or NULL */
+  const float* h_weight;       /* [width], and h_bias [width], or NULL */
+  const float* h_bias;
+  int32_t num_tokens, width, act_dtype;
+  float y_alpha, h_alpha;
+  int64_t x_stride_t, y_stride_t, base_stride_t;
+} hymeta_tanh_stream_args;
+int hymeta_tanh_stream(const hymeta_tanh_stream_args* args, hymeta_stream_t stream);
 
 #ifdef __cplusplus
 }

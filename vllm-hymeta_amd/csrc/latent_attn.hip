@@ -23,6 +23,14 @@ __device__ __forceinline__ void rotation_of(const double* freqs, int i, int turn
   }
 }
 
+// The two dimensions of the rotated part's pair i of `turning` that turn: (2 i, 2 i + 1), or split by half a rotated part
+// (i, i + turning); pairs behind them pass and are neighbours in both layouts.
+__device__ __forceinline__ void pair_at(int i, int turning, bool half, int* p, int* r) {
+  const bool split = half && i < turning;
+  *p = split ? i : 2 * i;
+  *r = split ? i + turning : 2 * i + 1;
+}
+
 __device__ __forceinline__ void fill_rotation(float* s_cos, float* s_sin, const double* freqs, int pairs, int turning, int pos, float mag) {
   for (int i = threadIdx.x; i < pairs; i += blockDim.x) rotation_of(freqs, i, turning, pos, mag, &s_cos[i], &s_sin[i]);
 }
@@ -69,7 +77,7 @@ __global__ __launch_bounds__(256) void latent_kv_prep_kernel(hymeta_latent_kv_pr
   const int s = seq_of_row(a.query_start_loc, a.num_seqs, t);
   const int pos = max(a.seq_lens[s] - (a.query_start_loc[s + 1] - t), 0);
   elem* row = static_cast<elem*>(a.proj) + static_cast<int64_t>(t) * a.proj_stride_t;
-  wave_rms_norm<A>(row + a.q_col, row + a.q_col, a.q_norm_weight, a.q_rank, a.eps, lane);         // the query latent, in place
+  if (a.q_rank > 0) wave_rms_norm<A>(row + a.q_col, row + a.q_col, a.q_norm_weight, a.q_rank, a.eps, lane);         // the query latent, in place
   const int64_t slot = a.slot_mapping ? a.slot_mapping[t] : -1;
   if (slot < 0 || slot >= a.num_blocks * a.block_size || a.kv_cache == nullptr) return;
   elem* dst = static_cast<elem*>(a.kv_cache) + slot * static_cast<int64_t>(a.kv_rank + a.rot_dim);
@@ -78,9 +86,11 @@ __global__ __launch_bounds__(256) void latent_kv_prep_kernel(hymeta_latent_kv_pr
   for (int i = lane; i < a.rot_dim / 2; i += 64) {
     float c, sn;
     rotation_of(a.rot_freqs, i, a.rot_dims / 2, pos, a.rot_mag, &c, &sn);
-    const float u = A::ld(kv + a.kv_rank + 2 * i), v = A::ld(kv + a.kv_rank + 2 * i + 1);
-    A::st(dst + a.kv_rank + 2 * i, u * c - v * sn);
-    A::st(dst + a.kv_rank + 2 * i + 1, v * c + u * sn);
+    int p, r;
+    pair_at(i, a.rot_dims / 2, a.rot_half != 0, &p, &r);
+    const float u = A::ld(kv + a.kv_rank + p), v = A::ld(kv + a.kv_rank + r);
+    A::st(dst + a.kv_rank + p, u * c - v * sn);
+    A::st(dst + a.kv_rank + r, v * c + u * sn);
   }
 }
 
@@ -106,9 +116,11 @@ __global__ __launch_bounds__(256) void latent_q_assemble_kernel(hymeta_latent_q_
     } else {
       const int i = j - C;
       const elem* qr = q + static_cast<int64_t>(h) * (a.dim + a.rot_dim) + a.dim;
-      const float u = A::ld(qr + 2 * i), v = A::ld(qr + 2 * i + 1);
-      A::st(o + C + 2 * i, u * s_cos[i] - v * s_sin[i]);
-      A::st(o + C + 2 * i + 1, v * s_cos[i] + u * s_sin[i]);
+      int p, r;
+      pair_at(i, a.rot_dims / 2, a.rot_half != 0, &p, &r);
+      const float u = A::ld(qr + p), v = A::ld(qr + r);
+      A::st(o + C + p, u * s_cos[i] - v * s_sin[i]);
+      A::st(o + C + r, v * s_cos[i] + u * s_sin[i]);
     }
   }
 }
@@ -122,18 +134,18 @@ using namespace hymeta;
 extern "C" int hymeta_latent_kv_prep(const hymeta_latent_kv_prep_args* args, hymeta_stream_t stream) {
   if (!args_ok(args)) return HYMETA_ERR_INVALID_ARG;
   const hymeta_latent_kv_prep_args& a = *args;
-  if (a.num_tokens < 0 || a.num_seqs < 0 || a.q_rank <= 0 || a.kv_rank <= 0 || a.rot_dim < 0 || a.rot_dims < 0 || a.q_col < 0 ||
+  if (a.num_tokens < 0 || a.num_seqs < 0 || a.q_rank < 0 || a.kv_rank <= 0 || a.rot_dim < 0 || a.rot_dims < 0 || a.q_col < 0 ||
       a.kv_col < 0 || a.block_size <= 0 || a.num_blocks < 0)
     return HYMETA_ERR_INVALID_ARG;
   if (a.rot_dim % 2 != 0 || a.rot_dims % 2 != 0 || a.rot_dims > a.rot_dim) return HYMETA_ERR_INVALID_ARG;
   if (!act_dtype_ok(a.act_dtype)) return HYMETA_ERR_UNSUPPORTED;
   if (a.rot_dim / 2 > kMaxRotPairs) return HYMETA_ERR_UNSUPPORTED;
   if (a.num_tokens == 0 || a.num_seqs == 0) return HYMETA_OK;
-  if (!a.proj || !a.q_norm_weight || !a.kv_norm_weight || !a.query_start_loc || !a.seq_lens || (a.rot_dims > 0 && !a.rot_freqs))
+  if (!a.proj || (a.q_rank > 0 && !a.q_norm_weight) || !a.kv_norm_weight || !a.query_start_loc || !a.seq_lens || (a.rot_dims > 0 && !a.rot_freqs))
     return HYMETA_ERR_INVALID_ARG;
   if (a.slot_mapping && !a.kv_cache) return HYMETA_ERR_INVALID_ARG;
   if (a.proj_stride_t < a.q_col + a.q_rank || a.proj_stride_t < a.kv_col + a.kv_rank + a.rot_dim) return HYMETA_ERR_INVALID_ARG;
-  const bool apart = a.q_col + a.q_rank <= a.kv_col || a.kv_col + a.kv_rank + a.rot_dim <= a.q_col;
+  const bool apart = a.q_rank == 0 || a.q_col + a.q_rank <= a.kv_col || a.kv_col + a.kv_rank + a.rot_dim <= a.q_col;
   if (!apart) return HYMETA_ERR_INVALID_ARG;
   hipStream_t st = begin_launches(stream);
   if (a.act_dtype == HYMETA_BF16) hipLaunchKernelGGL(latent_kv_prep_kernel<ActBf16>, dim3((a.num_tokens + 3) / 4), dim3(256), 0, st, a);

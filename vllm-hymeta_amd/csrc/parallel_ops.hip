@@ -1,6 +1,6 @@
 // Glue of parallel-layer designs (one norm, mixer and feed-forward side by side on an fp32 stream): the sum of a
-// layer's outputs onto the stream with the next layer's scalar-weight RMS norm; the rotate-half rotation of a fused
-// projection's queries and keys with the paged key / value write; and the short causal convolution (bias, silu) of a
+// layer's outputs onto the stream with the next layer's scalar-weight RMS norm; the rotation (in either pair layout, with
+// or without heads of unit root mean square) of a fused projection's queries and keys with the paged key / value write; and the short causal convolution (bias, silu) of a
 // state-space layer with its step sizes.  act_dtype in and out, fp32 inside.
 #include "act_types.h"
 
@@ -146,6 +146,124 @@ __global__ __launch_bounds__(256) void rotary_cache_kernel(hymeta_rotary_cache_a
       const int g = w / Dv, d = w % Dv;
       cache[static_cast<int64_t>(g) * (D + Dv) + D + d] = vsrc[w];
     }
+  }
+}
+
+// Pairs in either layout, cos and sin times a factor, and heads of unit root mean square.  grid = tokens, 256 threads;
+// `lanes` neighbouring lanes (a power of two) share a head.  Vec (interleaved pairs, heads and rows in whole eights): a lane
+// keeps 8 consecutive elements, read once; otherwise the lanes stride over the head's pairs and passing dimensions.  The
+// mean of squares is taken ahead of the turn: a pair's turn leaves u^2 + v^2 but for mag^2.
+template <typename A, bool Vec>
+__global__ __launch_bounds__(256) void rotary_unit_cache_kernel(hymeta_rotary_cache_args a, int lanes) {
+  typedef typename A::elem elem;
+  __shared__ __attribute__((aligned(16))) float s_cos[kMaxRotPairs], s_sin[kMaxRotPairs];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int H = a.num_heads, G = a.num_kv_heads, D = a.head_dim, Dv = a.v_dim, half = a.rot_dims / 2;
+  int pos;
+  if (a.positions) {
+    pos = static_cast<int>(a.positions[t]);
+  } else {
+    const int s = seq_of_row(a.query_start_loc, a.num_seqs, t);
+    pos = max(a.seq_lens[s] - (a.query_start_loc[s + 1] - t), 0);
+  }
+  const float mag = a.rot_mag != 0.f ? a.rot_mag : 1.f, mag2 = mag * mag;
+  for (int i = tid; i < half; i += 256) {
+    constexpr double kTwoPi = 6.283185307179586476925286766559, kInvTwoPi = 0.15915494309189533576888376337251;
+    const double ang = static_cast<double>(pos) * a.rot_freqs[i];
+    const float r = static_cast<float>(fma(-kTwoPi, rint(ang * kInvTwoPi), ang));
+    s_cos[i] = cosf(r) * mag;
+    s_sin[i] = sinf(r) * mag;
+  }
+  __syncthreads();
+  elem* row = static_cast<elem*>(a.qkv) + static_cast<int64_t>(t) * a.qkv_stride_t;
+  const int64_t slot = a.slot_mapping ? a.slot_mapping[t] : -1;
+  const bool store = a.kv_cache != nullptr && slot >= 0 && slot < a.num_blocks * a.block_size;
+  elem* cache = store ? static_cast<elem*>(a.kv_cache) + slot * G * static_cast<int64_t>(D + Dv) : nullptr;
+  const float ks = a.k_scale != 0.f ? a.k_scale : 1.f;
+  const int sub = tid & (lanes - 1), first = tid / lanes, step = 256 / lanes;
+  for (int head = first; head < H + G; head += step) {
+    const bool is_q = head < H;
+    elem* src = row + static_cast<int64_t>(head) * D;
+    elem* dst = (is_q || !cache) ? nullptr : cache + static_cast<int64_t>(head - H) * (D + Dv);
+    float ss = 0.f, v[8];
+    const bool on = 8 * sub < D, turns = 8 * sub < a.rot_dims;
+    if (Vec) {
+      if (on) A::ld4(src + 8 * sub, v), A::ld4(src + 8 * sub + 4, v + 4);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss = on ? fmaf(v[e], v[e], ss) : ss;
+      if (turns) ss *= mag2;
+    } else if (a.unit_rms) {
+      for (int d = sub; d < D; d += lanes) {
+        const float x = A::ld(src + d);
+        ss = fmaf(d < a.rot_dims ? x * mag2 : x, x, ss);
+      }
+    }
+    float mul = is_q ? 1.f : ks;
+    if (a.unit_rms) {
+      for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+      mul /= sqrtf(ss / static_cast<float>(D) + a.unit_eps);
+    }
+    if (Vec) {
+      if (!on) continue;
+      if (turns) {
+        const f32x4 c = *reinterpret_cast<const f32x4*>(s_cos + 4 * sub), sn = *reinterpret_cast<const f32x4*>(s_sin + 4 * sub);
+#pragma unroll
+        for (int p = 0; p < 4; ++p) {
+          const float u = v[2 * p], w = v[2 * p + 1];
+          v[2 * p] = u * c[p] - w * sn[p];
+          v[2 * p + 1] = w * c[p] + u * sn[p];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] *= mul;
+      A::st4(src + 8 * sub, v), A::st4(src + 8 * sub + 4, v + 4);
+      if (dst) A::st4(dst + 8 * sub, v), A::st4(dst + 8 * sub + 4, v + 4);
+    } else {
+      for (int i = sub; i < half; i += lanes) {
+        const int p = a.interleaved ? 2 * i : i, r = a.interleaved ? 2 * i + 1 : i + half;
+        const float u = A::ld(src + p), w = A::ld(src + r), c = s_cos[i], sn = s_sin[i];
+        const float ru = (u * c - w * sn) * mul, rw = (w * c + u * sn) * mul;
+        A::st(src + p, ru);
+        A::st(src + r, rw);
+        if (dst) {
+          A::st(dst + p, ru);
+          A::st(dst + r, rw);
+        }
+      }
+      for (int d = a.rot_dims + sub; d < D; d += lanes) {
+        const float x = A::ld(src + d) * mul;
+        A::st(src + d, x);
+        if (dst) A::st(dst + d, x);
+      }
+    }
+  }
+  if (cache) {
+    const elem* vsrc = row + static_cast<int64_t>(H + G) * D;
+    if (Vec) {
+      for (int w = 4 * tid; w < G * Dv; w += 4 * 256) {
+        float x[4];
+        A::ld4(vsrc + w, x);
+        A::st4(cache + static_cast<int64_t>(w / Dv) * (D + Dv) + D + w % Dv, x);
+      }
+    } else {
+      for (int w = tid; w < G * Dv; w += 256) cache[static_cast<int64_t>(w / Dv) * (D + Dv) + D + w % Dv] = vsrc[w];
+    }
+  }
+}
+
+template <typename A>
+void launch_rotary_unit(const hymeta_rotary_cache_args& a, hipStream_t st) {
+  const int bytes = A::kDtype == HYMETA_BF16 ? 2 : 4;
+  auto fours = [&](const void* p) { return reinterpret_cast<uintptr_t>(p) % (4 * bytes) == 0; };
+  const bool vec = (a.interleaved || a.rot_dims == 0) && a.head_dim % 8 == 0 && a.head_dim <= 512 && a.rot_dims % 8 == 0 && a.v_dim % 4 == 0 &&
+                   a.qkv_stride_t % 4 == 0 && fours(a.qkv) && fours(a.kv_cache);
+  int lanes = 64;
+  if (vec) {
+    lanes = 1;
+    while (8 * lanes < a.head_dim) lanes *= 2;
+    hipLaunchKernelGGL((rotary_unit_cache_kernel<A, true>), dim3(a.num_tokens), dim3(256), 0, st, a, lanes);
+  } else {
+    hipLaunchKernelGGL((rotary_unit_cache_kernel<A, false>), dim3(a.num_tokens), dim3(256), 0, st, a, lanes);
   }
 }
 
@@ -349,7 +467,13 @@ extern "C" int hymeta_rotary_cache(const hymeta_rotary_cache_args* args, hymeta_
   if (a.kv_cache && (!a.slot_mapping || a.block_size <= 0)) return HYMETA_ERR_INVALID_ARG;
   if (a.qkv_stride_t < static_cast<int64_t>(a.num_heads + a.num_kv_heads) * a.head_dim + (a.kv_cache ? static_cast<int64_t>(a.num_kv_heads) * a.v_dim : 0))
     return HYMETA_ERR_INVALID_ARG;
+  if (a.unit_rms && a.unit_eps < 0.f) return HYMETA_ERR_INVALID_ARG;
   hipStream_t st = begin_launches(stream);
+  if (a.interleaved || a.unit_rms || (a.rot_mag != 0.f && a.rot_mag != 1.f)) {
+    if (a.act_dtype == HYMETA_BF16) launch_rotary_unit<ActBf16>(a, st);
+    else launch_rotary_unit<ActF32>(a, st);
+    return launch_status();
+  }
   if (a.act_dtype == HYMETA_BF16) hipLaunchKernelGGL(rotary_cache_kernel<ActBf16>, dim3(a.num_tokens), dim3(256), 0, st, a);
   else hipLaunchKernelGGL(rotary_cache_kernel<ActF32>, dim3(a.num_tokens), dim3(256), 0, st, a);
   return launch_status();

@@ -138,6 +138,14 @@ __device__ __forceinline__ float distance_bias(int mode, float a, float b, int d
   return mode == HYMETA_BIAS_LOG_DISTANCE ? a * log1pf(b * static_cast<float>(dist)) : 0.f;
 }
 
+// First key a query at position pos sees: `window_left` tokens back, or the start of its chunk of `chunk` tokens (counted from
+// the sequence's first token), or the sequence's first.  Never decreases with pos.
+__host__ __device__ __forceinline__ bool bounded(const hymeta_sink_attention_args& a) { return a.window_left >= 0 || a.chunk > 0; }
+__device__ __forceinline__ int first_key(const hymeta_sink_attention_args& a, int pos) {
+  if (a.chunk > 0) return pos / a.chunk * a.chunk;
+  return a.window_left >= 0 ? max(0, pos - a.window_left) : 0;
+}
+
 // One wave per (query row, head).  Keys in tiles of 64: lane = key for the scores, lane = value channel for the
 // weighted sum, the tile's weights and row addresses handed over through LDS.
 template <typename A>
@@ -152,7 +160,7 @@ __global__ __launch_bounds__(64) void sink_attention_rows_kernel(hymeta_sink_att
   const int s = seq_of_row(a.query_start_loc, a.num_seqs, t);
   const int pos = a.seq_lens[s] - (a.query_start_loc[s + 1] - t);
   if (pos < 0) return;
-  const int first = a.window_left >= 0 ? max(0, pos - a.window_left) : 0;
+  const int first = first_key(a, pos);
   const elem* q = static_cast<const elem*>(a.q) + static_cast<int64_t>(t) * a.q_stride_t + static_cast<int64_t>(h) * D;
   for (int d = lane; d < D; d += 64) s_q[d] = A::ld(q + d);
   const int32_t* bt = a.block_tables + static_cast<int64_t>(s) * a.block_table_stride;
@@ -410,6 +418,7 @@ struct WaveRows {
   f32x4v o[RB][DV / 16];
   float m[RB], l[RB];          // running maximum of the row; this lane's share of the denominator
   int pos[RB];                 // position of the row's query (-1: no such row)
+  int first[RB];               // the first key it sees
   float ba[RB], bb[RB];
 };
 
@@ -474,8 +483,7 @@ __device__ __forceinline__ void attend_tile(WaveRows<D, DV, RB>& w, const MfmaSm
         }
         if (Masked) {
           const int j = j0 + 16 * (ks_lo + ks) + 4 * g4 + r;
-          const int first = a.window_left >= 0 ? pos - a.window_left : 0;
-          sc = (j <= pos && (j >= first || j < a.keep_first)) ? sc : -INFINITY;
+          sc = (j <= pos && (j >= w.first[rb] || j < a.keep_first)) ? sc : -INFINITY;
         }
         s[rb][ks][r] = sc;
         mx = fmaxf(mx, sc);
@@ -547,12 +555,11 @@ __device__ __forceinline__ void load_q(WaveRows<D, DV, RB>& w, int rb, const uin
     w.q[rb][st] = qrow ? __builtin_bit_cast(bf16x8, ld16g(qrow + 32 * st + 8 * g4)) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
 }
 
-// Whether every key of the tile from j0 on is visible to every query position in [p_lo, p_hi] / none of them to any.
-__device__ __forceinline__ bool tile_open(const hymeta_sink_attention_args& a, int j0, int p_lo, int p_hi) {
-  return j0 + kTileKeys - 1 <= p_lo && (a.window_left < 0 || j0 >= p_hi - a.window_left);
-}
-__device__ __forceinline__ bool tile_shut(const hymeta_sink_attention_args& a, int j0, int p_lo) {
-  return a.window_left >= 0 && j0 + kTileKeys - 1 < p_lo - a.window_left && j0 >= a.keep_first;
+// Whether every key of the tile from j0 on is visible to every query position in [p_lo, p_hi] (first_hi: the first key p_hi
+// sees) / none of them to any (first_lo: the first key p_lo sees).
+__device__ __forceinline__ bool tile_open(int j0, int p_lo, int first_hi) { return j0 + kTileKeys - 1 <= p_lo && j0 >= first_hi; }
+__device__ __forceinline__ bool tile_shut(const hymeta_sink_attention_args& a, int j0, int first_lo) {
+  return j0 + kTileKeys - 1 < first_lo && j0 >= a.keep_first;
 }
 
 // The bias' constants of head h as attend_tile wants them.
@@ -594,6 +601,7 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
     const int r = wrow + 16 * rb + n;
     const bool ok = r < q;
     w.pos[rb] = ok ? ctx + r : -1;
+    w.first[rb] = first_key(a, ctx + r);
     load_bias<D, DV, RB>(w, rb, a, h);
     w.m[rb] = a.sink ? (a.sink_logits ? a.sink_logits[h] * 1.4426950408889634f : 0.f) : -INFINITY;
     w.l[rb] = (a.sink && g4 == 0) ? 1.f : 0.f;        // the sink's exp(m - m), counted once per row
@@ -603,10 +611,10 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
   }
   const int block_last = ctx + min(q, static_cast<int>(blockIdx.x) * kRows + kRows) - 1;      // last key any row of the block sees
   const int wave_last = ctx + min(q, wrow + 16 * RB) - 1;
-  int j_first = 0;
-  if (a.window_left >= 0) j_first = max(0, ctx + static_cast<int>(blockIdx.x) * kRows - a.window_left) / kTileKeys * kTileKeys;
+  const int first_lo = first_key(a, ctx + wrow), first_hi = first_key(a, wave_last);           // of the wave's rows
+  const int j_first = first_key(a, ctx + static_cast<int>(blockIdx.x) * kRows) / kTileKeys * kTileKeys;
   // the tiles of the kept first keys that lie before the window's first tile come first, then the window's
-  const int keep_end = a.window_left >= 0 ? min((a.keep_first + kTileKeys - 1) / kTileKeys * kTileKeys, j_first) : 0;
+  const int keep_end = bounded(a) ? min((a.keep_first + kTileKeys - 1) / kTileKeys * kTileKeys, j_first) : 0;
   const int j_start = keep_end > 0 ? 0 : j_first;
   auto next = [&](int j0) { return (j0 < keep_end && j0 + kTileKeys >= keep_end) ? j_first : j0 + kTileKeys; };
   // two LDS images: while the waves multiply tile t out of one, tile t + 1 goes into the other and the loads of tile
@@ -624,9 +632,9 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
       const int j1 = next(j0), j2 = next(j1);
       if (j1 <= block_last) stage.commit(sm[buf ^ 1], s_scale[buf ^ 1]);
       if (j2 <= block_last) stage.issue(a, bt, g, j2, block_last);
-      if (wrow < q && j0 <= wave_last && !tile_shut(a, j0, ctx + wrow)) {
+      if (wrow < q && j0 <= wave_last && !tile_shut(a, j0, first_lo)) {
         // tiles whose every key is visible to every row of the wave need no mask
-        if (tile_open(a, j0, ctx + wrow, wave_last)) attend_tile<D, DV, RB, 4, false, kScaled>(w, sm[buf], s_scale[buf], a, j0, 0);
+        if (tile_open(j0, ctx + wrow, first_hi)) attend_tile<D, DV, RB, 4, false, kScaled>(w, sm[buf], s_scale[buf], a, j0, 0);
         else attend_tile<D, DV, RB, 4, true, kScaled>(w, sm[buf], s_scale[buf], a, j0, 0);
       }
       __syncthreads();
@@ -637,8 +645,8 @@ __global__ __launch_bounds__(64 * PrefillWaves<D>::value) void sink_attention_pr
     for (int j0 = j_start; j0 <= block_last; j0 = next(j0)) {
       const bool more = next(j0) <= block_last;
       if (more) stage.issue(a, bt, g, next(j0), block_last);
-      if (wrow < q && j0 <= wave_last && !tile_shut(a, j0, ctx + wrow)) {
-        if (tile_open(a, j0, ctx + wrow, wave_last)) attend_tile<D, DV, RB, 4, false, kScaled>(w, sm[0], s_scale[0], a, j0, 0);
+      if (wrow < q && j0 <= wave_last && !tile_shut(a, j0, first_lo)) {
+        if (tile_open(j0, ctx + wrow, first_hi)) attend_tile<D, DV, RB, 4, false, kScaled>(w, sm[0], s_scale[0], a, j0, 0);
         else attend_tile<D, DV, RB, 4, true, kScaled>(w, sm[0], s_scale[0], a, j0, 0);
       }
       __syncthreads();
@@ -720,8 +728,9 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
   // With a window: the tiles of the kept first keys that lie before the window's first tile, then the window's tiles
   // (tiles wholly before the window are not read), dealt evenly over the splits.
   int kept_tiles = 0, window_from = 0, num_tiles = pos / kTileKeys + 1, per = tiles_per_split;
-  if (a.window_left >= 0) {
-    window_from = max(0, pos - a.window_left) / kTileKeys * kTileKeys;
+  const int first = first_key(a, pos);
+  if (bounded(a)) {
+    window_from = first / kTileKeys * kTileKeys;
     kept_tiles = min((a.keep_first + kTileKeys - 1) / kTileKeys * kTileKeys, window_from) / kTileKeys;
     num_tiles = kept_tiles + (pos - window_from) / kTileKeys + 1;
     per = (num_tiles + splits - 1) / splits;
@@ -740,6 +749,7 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
     const bool ok = r < HG;
     const int h = g * group + vs.h_first + (ok ? r : 0);
     w.pos[rb] = ok ? pos : -1;
+    w.first[rb] = first;
     load_bias<D, DV, RB>(w, rb, a, h);
     w.m[rb] = -INFINITY;
     w.l[rb] = 0.f;
@@ -763,7 +773,7 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
       if (v + 1 <= v_hi) stage.commit(sm[buf ^ 1], s_scale[buf ^ 1]);
       if (v + 2 <= v_hi) stage.issue(a, bt, g, tile(v + 2), pos);
       if (j0 + 16 * wave <= pos) {
-        if (tile_open(a, j0, pos, pos)) attend_tile<D, DV, RB, 1, false, kScaled>(w, sm[buf], s_scale[buf], a, j0, wave);
+        if (tile_open(j0, pos, first)) attend_tile<D, DV, RB, 1, false, kScaled>(w, sm[buf], s_scale[buf], a, j0, wave);
         else attend_tile<D, DV, RB, 1, true, kScaled>(w, sm[buf], s_scale[buf], a, j0, wave);
       }
       __syncthreads();
@@ -775,7 +785,7 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void sink_attention_decode_mfma_
       const bool more = v + 1 <= v_hi;
       if (more) stage.issue(a, bt, g, tile(v + 1), pos);
       if (j0 + 16 * wave <= pos) {
-        if (tile_open(a, j0, pos, pos)) attend_tile<D, DV, RB, 1, false, kScaled>(w, sm[0], s_scale[0], a, j0, wave);
+        if (tile_open(j0, pos, first)) attend_tile<D, DV, RB, 1, false, kScaled>(w, sm[0], s_scale[0], a, j0, wave);
         else attend_tile<D, DV, RB, 1, true, kScaled>(w, sm[0], s_scale[0], a, j0, wave);
       }
       __syncthreads();
@@ -898,11 +908,11 @@ inline bool mfma_shape(const hymeta_sink_attention_args& a) {
          (reinterpret_cast<uintptr_t>(a.q) | reinterpret_cast<uintptr_t>(a.kv_cache) | reinterpret_cast<uintptr_t>(a.out)) % 16 == 0;
 }
 
-// window_left >= 0: a row reads the kept first keys' tiles and the window's, however long the sequence is.
-inline int decode_splits(int num_seqs, int num_heads, int num_kv_heads, int max_seq_len, int window_left = -1, int keep_first = 0) {
+// span > 0 (a window's or a chunk's keys): a row reads the kept first keys' tiles and the span's, however long the sequence is.
+inline int decode_splits(int num_seqs, int num_heads, int num_kv_heads, int max_seq_len, int64_t span = 0, int keep_first = 0) {
   int tiles = (max_seq_len + kTileKeys - 1) / kTileKeys;
-  if (window_left >= 0) {
-    const int64_t seen = (static_cast<int64_t>(keep_first) + kTileKeys - 1) / kTileKeys + static_cast<int64_t>(window_left) / kTileKeys + 2;
+  if (span > 0) {
+    const int64_t seen = (static_cast<int64_t>(keep_first) + kTileKeys - 1) / kTileKeys + (span - 1) / kTileKeys + 2;
     if (seen < tiles) tiles = static_cast<int>(seen);
   }
   // Workgroups aimed at: a workgroup's fixed cost (query fragments, first tile, the merge of its waves, its partial) grows
@@ -924,7 +934,7 @@ int launch_mfma(const hymeta_sink_attention_args& a, hipStream_t st, ValueSlice 
     hipLaunchKernelGGL((sink_attention_prefill_mfma_kernel<D, DV, kRB, Layout>), grid, dim3(64 * PrefillWaves<D>::value), 0, st, a, vs);
   }
   // sequences with a single row: every step but a pure prompt step has some; a prompt of one token is one too
-  const int splits = decode_splits(a.num_seqs, a.num_heads, a.num_kv_heads, a.max_seq_len, a.window_left, a.keep_first);
+  const int splits = decode_splits(a.num_seqs, a.num_heads, a.num_kv_heads, a.max_seq_len, a.chunk > 0 ? a.chunk : static_cast<int64_t>(a.window_left) + 1, a.keep_first);
   const int tiles = (a.max_seq_len + kTileKeys - 1) / kTileKeys;
   const int tiles_per_split = (tiles + splits - 1) / splits;
   const dim3 grid = Layout == HYMETA_KV_SHARED_KEY ? dim3((splits * a.num_seqs + 7) / 8 * 8 * a.num_kv_heads) : dim3(splits, a.num_kv_heads, a.num_seqs);
@@ -1017,6 +1027,7 @@ extern "C" int hymeta_sink_attention(const hymeta_sink_attention_args* args, hym
   if (a.kv_layout < HYMETA_KV_KEY_THEN_VALUE || a.kv_layout > HYMETA_KV_SCALED_KEY) return HYMETA_ERR_UNSUPPORTED;
   if (a.kv_layout == HYMETA_KV_SCALED_KEY && (a.v_dim != a.head_dim || reinterpret_cast<uintptr_t>(a.kv_cache) % 16 != 0)) return HYMETA_ERR_INVALID_ARG;
   if (a.window_left >= 0 && a.keep_first < 0) return HYMETA_ERR_INVALID_ARG;
+  if (a.chunk < 0 || (a.chunk > 0 && (a.window_left >= 0 || a.keep_first != 0))) return HYMETA_ERR_INVALID_ARG;
   if (a.kv_layout == HYMETA_KV_VALUE_IN_KEY && a.v_dim > a.head_dim) return HYMETA_ERR_INVALID_ARG;
   if (a.num_tokens == 0 || a.num_seqs == 0) return HYMETA_OK;
   if (!a.q || !a.kv_cache || !a.out || !a.block_tables || !a.query_start_loc || !a.seq_lens) return HYMETA_ERR_INVALID_ARG;

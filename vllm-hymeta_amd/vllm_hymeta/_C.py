@@ -42,7 +42,7 @@ MAX_STREAMS = 16
 LIGHTNING_CHUNK = 64
 CONV_MAX_TAPS = 8
 
-ABI_VERSION = 8
+ABI_VERSION = 9
 ERR_SCRATCH_LIMIT = -5
 GEMM_TICKET_BYTES = 16384
 STATIC_SCRATCH_BYTES = 16 << 20
@@ -369,6 +369,7 @@ class SinkAttentionArgs(_Args):
         ("sink_logits", _ptr), ("kv_layout", _i32), ("keep_first", _i32),
         ("softcap", _f32), ("head_gate", _ptr), ("head_gate_stride_t", _i64),
         ("elem_gate", _ptr), ("elem_gate_stride_t", _i64),
+        ("chunk", _i32),
     ]
 
 
@@ -431,6 +432,7 @@ class LatentKvPrepArgs(_Args):
         ("q_col", _i32), ("kv_col", _i32), ("block_size", _i32), ("act_dtype", _i32),
         ("eps", _f32), ("rot_mag", _f32),
         ("num_blocks", _i64), ("proj_stride_t", _i64),
+        ("rot_half", _i32),
     ]
 
 
@@ -442,6 +444,7 @@ class LatentQAssembleArgs(_Args):
         ("kv_rank", _i32), ("act_dtype", _i32),
         ("rot_mag", _f32),
         ("q_stride_t", _i64),
+        ("rot_half", _i32),
     ]
 
 
@@ -547,6 +550,19 @@ class RotaryCacheArgs(_Args):
         ("rot_dims", _i32), ("block_size", _i32), ("act_dtype", _i32),
         ("k_scale", _f32),
         ("num_blocks", _i64), ("qkv_stride_t", _i64),
+        ("interleaved", _i32), ("unit_rms", _i32),
+        ("rot_mag", _f32), ("unit_eps", _f32),
+    ]
+
+
+class TanhStreamArgs(_Args):
+    _fields_ = [
+        _SIZE,
+        ("x", _ptr), ("y", _ptr), ("y_weight", _ptr), ("y_bias", _ptr), ("base", _ptr), ("base2", _ptr), ("add", _ptr),
+        ("h_out", _ptr), ("h_weight", _ptr), ("h_bias", _ptr),
+        ("num_tokens", _i32), ("width", _i32), ("act_dtype", _i32),
+        ("y_alpha", _f32), ("h_alpha", _f32),
+        ("x_stride_t", _i64), ("y_stride_t", _i64), ("base_stride_t", _i64),
     ]
 
 
@@ -690,6 +706,7 @@ _SIGNATURES = {
     "hymeta_talk_qkv_prep": (C.c_int, [C.POINTER(TalkQkvPrepArgs), _ptr]),
     "hymeta_stream_add_norm": (C.c_int, [C.POINTER(StreamAddNormArgs), _ptr]),
     "hymeta_rotary_cache": (C.c_int, [C.POINTER(RotaryCacheArgs), _ptr]),
+    "hymeta_tanh_stream": (C.c_int, [C.POINTER(TanhStreamArgs), _ptr]),
     "hymeta_causal_conv": (C.c_int, [C.POINTER(CausalConvArgs), _ptr]),
     "hymeta_decay_scan_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32]),
     "hymeta_decay_scan": (C.c_int, [C.POINTER(DecayScanArgs), _ptr]),
@@ -743,6 +760,7 @@ STRUCTS = {
     "hymeta_decay_scan_args": DecayScanArgs,
     "hymeta_scaled_key_cache_args": ScaledKeyCacheArgs,
     "hymeta_delta_rule_args": DeltaRuleArgs,
+    "hymeta_tanh_stream_args": TanhStreamArgs,
 }
 
 

@@ -1654,13 +1654,14 @@ def sink_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_tables: torch.
                    bias_b: Optional[torch.Tensor] = None, sink: bool = True, window_left: int = -1,
                    sink_logits: Optional[torch.Tensor] = None, value_in_key: bool = False, shared_key: bool = False,
                    keep_first: int = 0, softcap: float = 0.0, head_gate: Optional[torch.Tensor] = None, scaled_key: bool = False,
-                   slopes: Optional[torch.Tensor] = None, elem_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   slopes: Optional[torch.Tensor] = None, elem_gate: Optional[torch.Tensor] = None, chunk: int = 0) -> torch.Tensor:
     """Causal attention of the rows ``q [T, H, D]`` over their sequences' paged keys (this step's included):
     ``softmax`` over ``scale q.k - bias_a[h] ln(1 + bias_b[h] (i - j))`` with, for ``sink``, ``exp(sink_logits[h])`` (one
     without ``sink_logits``) added to the denominator.  ``softcap > 0``: ``scale q.k`` becomes ``softcap tanh(scale q.k /
     softcap)``.  ``head_gate [T, H]`` (a view with any row stride): head ``h``'s output is multiplied by its sigmoid;
     ``elem_gate [T, H Dv]``: the output is multiplied by its sigmoid element by element.  ``slopes [H]`` (in place of ``bias_a`` /
-    ``bias_b``): the bias is ``slopes[h] (i - j)``.  ``scaled_key``: cache rows as ``scaled_key_cache_`` writes them.  ``value_in_key``: a cache row holds ``D`` elements per key/value
+    ``bias_b``): the bias is ``slopes[h] (i - j)``.  ``chunk > 0`` (in place of ``window_left``): a query sees the keys of its own run of
+    ``chunk`` positions, counted from the sequence's first token.  ``scaled_key``: cache rows as ``scaled_key_cache_`` writes them.  ``value_in_key``: a cache row holds ``D`` elements per key/value
     head, the first ``Dv`` of which are also the value (a latent that keys and values share).  Returns ``[T, H, Dv]``."""
     _dev(q, kv_cache, block_tables, query_start_loc, seq_lens, bias_a, bias_b, sink_logits, slopes, elem_gate)
     _require(q.dim() == 3 and q.stride(2) == 1 and q.stride(1) == head_dim and q.shape[2] == head_dim, "q must be [T, H, D] with contiguous heads")
@@ -1675,6 +1676,7 @@ def sink_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_tables: torch.
     _require(kv_cache.dtype == q.dtype and kv_cache.is_contiguous() and kv_cache.dim() == 4
              and kv_cache.shape[2:] == cache_tail, f"kv_cache must be contiguous [blocks, block_size, {cache_tail[0]}, {cache_tail[1]}]")
     _require(keep_first >= 0, "keep_first counts tokens")
+    _require(chunk >= 0 and (chunk == 0 or (window_left < 0 and keep_first == 0)), "a chunk goes without a window and kept first keys")
     _f32vec(sink_logits, H, "sink_logits")
     S = query_start_loc.numel() - 1
     _i32vec(query_start_loc, S + 1, "query_start_loc")
@@ -1704,7 +1706,7 @@ def sink_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_tables: torch.
         _require(elem_gate.shape == (T, H * v_dim) and elem_gate.stride(1) == 1 and elem_gate.dtype == q.dtype, "elem_gate must be [T, H Dv] of q's type with contiguous rows")
         a.elem_gate, a.elem_gate_stride_t = _p(elem_gate), elem_gate.stride(0)
     a.sink, a.window_left, a.max_query_len, a.max_seq_len, a.scale = int(bool(sink)), window_left, max_query_len, max_seq_len, scale
-    a.sink_logits, a.keep_first, a.softcap = _p(sink_logits), keep_first, float(softcap)
+    a.sink_logits, a.keep_first, a.softcap, a.chunk = _p(sink_logits), keep_first, float(softcap), int(chunk)
     if head_gate is not None:
         _dev(q, head_gate)
         _require(head_gate.shape == (T, H) and head_gate.stride(1) == 1 and head_gate.dtype == q.dtype, "head_gate must be [T, H] of q's type with contiguous heads")
@@ -1860,16 +1862,17 @@ def add_group_norm(x: torch.Tensor, y: Optional[torch.Tensor], weight: torch.Ten
 
 
 def latent_kv_prep_(proj: torch.Tensor, q_col: int, q_rank: int, kv_col: int, kv_rank: int, rot_dim: int, rot_dims: int,
-                    q_norm_weight: torch.Tensor, kv_norm_weight: torch.Tensor, eps: float, rot_freqs: torch.Tensor, rot_mag: float,
+                    q_norm_weight: Optional[torch.Tensor], kv_norm_weight: torch.Tensor, eps: float, rot_freqs: torch.Tensor, rot_mag: float,
                     kv_cache: Optional[torch.Tensor], slot_mapping: Optional[torch.Tensor], query_start_loc: torch.Tensor,
-                    seq_lens: torch.Tensor) -> None:
+                    seq_lens: torch.Tensor, rot_half: bool = False) -> None:
     """On the rows ``proj [T, ...]`` of the fused down projections: RMS norm of the query latent (columns ``q_col ..``) in
-    place; RMS norm of the key/value latent (columns ``kv_col ..``) and rotation of the ``rot_dim`` columns behind it,
-    both written to ``kv_cache [blocks, block_size, 1, kv_rank + rot_dim]`` at ``slot_mapping``."""
+    place (``q_rank`` 0: there is none); RMS norm of the key/value latent (columns ``kv_col ..``) and rotation of the ``rot_dim`` columns behind it
+    (neighbouring pairs, or with ``rot_half`` pairs ``(i, i + rot_dims / 2)``), both written to ``kv_cache [blocks, block_size, 1, kv_rank + rot_dim]`` at ``slot_mapping``."""
     _dev(proj, q_norm_weight, kv_norm_weight, rot_freqs, kv_cache, slot_mapping, query_start_loc, seq_lens)
     _require(proj.dim() == 2 and proj.stride(1) == 1, "proj must be row-contiguous")
     T = proj.shape[0]
     _require(q_col + q_rank <= proj.shape[1] and kv_col + kv_rank + rot_dim <= proj.shape[1], "the latents' columns must lie inside proj")
+    _require((q_norm_weight is None) == (q_rank == 0), "a query latent comes with its norm")
     _f32vec(q_norm_weight, q_rank, "q_norm_weight")
     _f32vec(kv_norm_weight, kv_rank, "kv_norm_weight")
     _require(rot_freqs.dtype == torch.float64 and rot_freqs.is_contiguous() and rot_freqs.numel() * 2 >= rot_dims, "rot_freqs must be float64 [rot_dims / 2]")
@@ -1880,7 +1883,7 @@ def latent_kv_prep_(proj: torch.Tensor, q_col: int, q_rank: int, kv_col: int, kv
     a.proj, a.q_norm_weight, a.kv_norm_weight, a.rot_freqs = _p(proj), _p(q_norm_weight), _p(kv_norm_weight), _p(rot_freqs)
     a.query_start_loc, a.seq_lens = _p(query_start_loc), _p(seq_lens)
     a.num_tokens, a.num_seqs, a.q_rank, a.kv_rank, a.rot_dim, a.rot_dims, a.q_col, a.kv_col = T, S, q_rank, kv_rank, rot_dim, rot_dims, q_col, kv_col
-    a.block_size, a.act_dtype, a.eps, a.rot_mag, a.proj_stride_t = 1, _act(proj), eps, rot_mag, proj.stride(0)
+    a.block_size, a.act_dtype, a.eps, a.rot_mag, a.proj_stride_t, a.rot_half = 1, _act(proj), eps, rot_mag, proj.stride(0), int(rot_half)
     if kv_cache is not None and kv_cache.numel() > 0 and slot_mapping is not None:
         _require(kv_cache.dtype == proj.dtype and kv_cache.is_contiguous() and kv_cache.dim() == 4 and kv_cache.shape[2:] == (1, kv_rank + rot_dim),
                  "kv_cache must be contiguous [blocks, block_size, 1, kv_rank + rot_dim]")
@@ -1890,7 +1893,7 @@ def latent_kv_prep_(proj: torch.Tensor, q_col: int, q_rank: int, kv_col: int, kv
 
 
 def latent_q_assemble(q: torch.Tensor, q_abs: torch.Tensor, dim: int, rot_dim: int, rot_dims: int, rot_freqs: torch.Tensor,
-                      rot_mag: float, query_start_loc: torch.Tensor, seq_lens: torch.Tensor) -> torch.Tensor:
+                      rot_mag: float, query_start_loc: torch.Tensor, seq_lens: torch.Tensor, rot_half: bool = False) -> torch.Tensor:
     """``q [T, H, dim + rot_dim]`` and ``q_abs [H, T, C]`` -> ``[T, H, C + rot_dim]``: the absorbed part followed by the
     rotated part of every head's query."""
     _dev(q, q_abs, rot_freqs, query_start_loc, seq_lens)
@@ -1906,7 +1909,7 @@ def latent_q_assemble(q: torch.Tensor, q_abs: torch.Tensor, dim: int, rot_dim: i
     a = _C.LatentQAssembleArgs()
     a.q, a.q_abs, a.out, a.rot_freqs, a.query_start_loc, a.seq_lens = _p(q), _p(q_abs), _p(out), _p(rot_freqs), _p(query_start_loc), _p(seq_lens)
     a.num_tokens, a.num_seqs, a.num_heads, a.dim, a.rot_dim, a.rot_dims, a.kv_rank, a.act_dtype = T, S, H, dim, rot_dim, rot_dims, Ck, _act(q)
-    a.rot_mag, a.q_stride_t = rot_mag, q.stride(0)
+    a.rot_mag, a.q_stride_t, a.rot_half = rot_mag, q.stride(0), int(rot_half)
     _C.check(_C.load().hymeta_latent_q_assemble(C.byref(a), _stream(q)), "hymeta_latent_q_assemble")
     return out
 
@@ -2303,9 +2306,11 @@ def stream_add_norm_(x: torch.Tensor, terms: Sequence[Tuple[torch.Tensor, float,
 def rotary_cache_(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, rot_dims: int,
                   rot_freqs: Optional[torch.Tensor], k_scale: float = 1.0, kv_cache: Optional[torch.Tensor] = None,
                   slot_mapping: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None,
-                  query_start_loc: Optional[torch.Tensor] = None, seq_lens: Optional[torch.Tensor] = None) -> None:
+                  query_start_loc: Optional[torch.Tensor] = None, seq_lens: Optional[torch.Tensor] = None, interleaved: bool = False,
+                  rot_mag: float = 1.0, unit_eps: Optional[float] = None) -> None:
     """On the rows ``qkv [T, H D + G D + G Dv (+ ...)]`` of a fused projection, in place: dimensions ``i`` and ``i + rot_dims / 2``
-    of every query and key head turn by ``position * rot_freqs[i]`` (``rot_freqs`` float64 ``[rot_dims / 2]``), keys are
+    (``interleaved``: ``2 i`` and ``2 i + 1``) of every query and key head turn by ``position * rot_freqs[i]`` (``rot_freqs`` float64
+    ``[rot_dims / 2]``), cos and sin times ``rot_mag``; with ``unit_eps`` every head is divided by its root mean square; keys are
     multiplied by ``k_scale``, and with ``kv_cache [blocks, block_size, G, D + Dv]`` the keys and values are written at
     ``slot_mapping``.  Positions: ``positions`` (int64) or the rows' places in their sequences (``query_start_loc``, ``seq_lens``)."""
     _dev(qkv, rot_freqs, kv_cache, slot_mapping, positions, query_start_loc, seq_lens)
@@ -2330,6 +2335,7 @@ def rotary_cache_(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim
     a.qkv, a.rot_freqs, a.positions = _p(qkv), _p(rot_freqs), _p(positions)
     a.num_tokens, a.num_heads, a.num_kv_heads, a.head_dim, a.v_dim, a.rot_dims = T, H, G, D, Dv, rot_dims
     a.act_dtype, a.k_scale, a.qkv_stride_t, a.block_size = _act(qkv), float(k_scale), qkv.stride(0), 1
+    a.interleaved, a.rot_mag, a.unit_rms, a.unit_eps = int(interleaved), float(rot_mag), int(unit_eps is not None), float(unit_eps or 0.0)
     if kv_cache is not None:
         _require(kv_cache.dtype == qkv.dtype and kv_cache.is_contiguous() and kv_cache.dim() == 4 and kv_cache.shape[2:] == (G, D + Dv),
                  "kv_cache must be contiguous [blocks, block_size, G, D + Dv]")
@@ -2478,3 +2484,50 @@ def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, beta_logit: to
         a.workspace, a.workspace_bytes = _p(ws), ws.numel()
     _C.check(lib.hymeta_delta_rule(C.byref(a), _stream(q)), "hymeta_delta_rule")
     return out
+
+
+# =============================================================================================== squashing norms
+class SquashNorm(NamedTuple):
+    """``tanh(alpha v) weight + bias``, element by element."""
+    alpha: float
+    weight: torch.Tensor          # fp32 [W]
+    bias: torch.Tensor            # fp32 [W]
+
+
+def tanh_stream_(x: torch.Tensor, y: Optional[torch.Tensor] = None, y_norm: Optional[SquashNorm] = None, base: Optional[torch.Tensor] = None,
+                 base2: Optional[torch.Tensor] = None, add: Optional[torch.Tensor] = None, read: Optional[SquashNorm] = None,
+                 out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+    """On the fp32 stream ``x [T, W]``, in place, one launch: ``x = base (+ base2) (+ add)`` with ``base`` (fp32 ``[T, W]``), then
+    ``x += y_norm(y)`` with ``y``.  ``out_dtype``: returns ``read(x)`` (without ``read``: ``x``) in that type."""
+    _dev(x, y, base, base2, add, *(t for n in (y_norm, read) if n is not None for t in (n.weight, n.bias)))
+    _require(x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1, "x must be row-contiguous fp32 [T, W]")
+    _require((y is None) == (y_norm is None), "y comes with its norm")
+    _require(y is not None or base is not None or out_dtype is not None, "nothing to do")
+    T, W = x.shape
+    a = _C.TanhStreamArgs()
+    a.x, a.num_tokens, a.width, a.x_stride_t = _p(x), T, W, x.stride(0)
+    act = y.dtype if y is not None else (out_dtype or torch.float32)
+    _require(out_dtype is None or out_dtype == act, "the sublayers' activations have one type")
+    _require(act in _DT, "activations must be bf16 or fp32")
+    a.act_dtype = _DT[act]
+    if y is not None:
+        _require(y.shape == (T, W) and y.stride(1) == 1, "y must be row-contiguous [T, W]")
+        _f32vec(y_norm.weight, W, "y_norm.weight"), _f32vec(y_norm.bias, W, "y_norm.bias")
+        a.y, a.y_stride_t, a.y_alpha, a.y_weight, a.y_bias = _p(y), y.stride(0), float(y_norm.alpha), _p(y_norm.weight), _p(y_norm.bias)
+    if base is not None:
+        for b in (base, base2):
+            _require(b is None or (b.shape == (T, W) and b.dtype == torch.float32 and b.stride(1) == 1 and b.stride(0) == base.stride(0)),
+                     "base and base2 must be row-contiguous fp32 [T, W] of one stride")
+        _f32vec(add, W, "add")
+        a.base, a.base2, a.add, a.base_stride_t = _p(base), _p(base2), _p(add), base.stride(0)
+    else:
+        _require(base2 is None and add is None, "base2 and add come with base")
+    h = None
+    if out_dtype is not None:
+        h = torch.empty(T, W, dtype=out_dtype, device=x.device)
+        a.h_out = _p(h)
+        if read is not None:
+            _f32vec(read.weight, W, "read.weight"), _f32vec(read.bias, W, "read.bias")
+            a.h_weight, a.h_bias, a.h_alpha = _p(read.weight), _p(read.bias), float(read.alpha)
+    _C.check(_C.load().hymeta_tanh_stream(C.byref(a), _stream(x)), "hymeta_tanh_stream")
+    return h

@@ -163,3 +163,13 @@ class LinearColumns(torch.nn.Module):
     def forward(self, x: torch.Tensor, defer: bool = False) -> torch.Tensor:
         return self.parent(x)[:, self.lo:self.hi]
 
+
+
+def linear_fp32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """``x W^T`` with an fp32 result that is not rounded to the activations' type: products that become an fp32 stream.
+    bf16: the weight-streaming kernels for decode-sized batches, else the library GEMM with an fp32 output."""
+    if x.dtype != torch.bfloat16:
+        return torch.nn.functional.linear(x, weight)
+    if x.shape[0] <= hip_ops.BF16_GEMM_TALL_ROWS and hip_ops.logits_supported(x, weight):
+        return hip_ops.bf16_logits(x, weight)
+    return torch.mm(x, weight.t(), out_dtype=torch.float32)

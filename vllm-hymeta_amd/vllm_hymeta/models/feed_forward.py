@@ -76,7 +76,10 @@ class SiluGluMLP(torch.nn.Module):
         self.gate_up_proj, self.down_proj = gate_up_proj, down_proj
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
-        return self.down_proj(hip_ops.silu_mul(self.gate_up_proj(h)))
+        gu = self.gate_up_proj
+        if gu.bias is None and hip_ops.gemm_silu_mul_supported(h, gu.weight):      # decode-sized bf16 batches: in the GEMM's epilogue
+            return self.down_proj(hip_ops.gemm_silu_mul(h, gu.weight))
+        return self.down_proj(hip_ops.silu_mul(gu(h)))
 
 
 class GeluGluMLP(torch.nn.Module):

@@ -27,7 +27,7 @@ class StepLayout:
     query_start_loc: torch.Tensor
     context_lens: torch.Tensor
     seq_lens: torch.Tensor
-    slot_idx: torch.Tensor
+    slot_idx: Optional[torch.Tensor]              # None: the model carries no recurrent state
     block_tables: Optional[torch.Tensor]
     slot_mapping: Optional[torch.Tensor]
     max_query_len: int

@@ -41,6 +41,11 @@ def _nilevik_config(model_dir: str):
     return NilevikConfig.from_pretrained(model_dir)
 
 
+def _banitar_config(model_dir: str):
+    from .models.configuration_banitar import BanitarConfig
+    return BanitarConfig.from_pretrained(model_dir)
+
+
 def _gla_swa_config(model_dir: str):
     from .model_for_7B.configuration_gla_swa import GLAswaConfig
     with open(os.path.join(model_dir, "config.json")) as f:
@@ -59,6 +64,8 @@ register("Dapuzen", "vllm_hymeta.models.modeling_dapuzen:DapuzenForCausalLM", _d
 register("DapuzenForCausalLM", "vllm_hymeta.models.modeling_dapuzen:DapuzenForCausalLM", _dapuzen_config)
 register("Nilevik", "vllm_hymeta.models.modeling_nilevik:NilevikForCausalLM", _nilevik_config)
 register("NilevikForCausalLM", "vllm_hymeta.models.modeling_nilevik:NilevikForCausalLM", _nilevik_config)
+register("Banitar", "vllm_hymeta.models.modeling_banitar:BanitarForCausalLM", _banitar_config)
+register("BanitarForCausalLM", "vllm_hymeta.models.modeling_banitar:BanitarForCausalLM", _banitar_config)
 register("GLAswaForCausalLM", "vllm_hymeta.model_for_7B.modeling_gla_swa:GLAswaForCausalLM", _gla_swa_config)
 
 
@@ -95,6 +102,8 @@ _KERNEL_SOURCES = {
     "DapuzenForCausalLM": ("api_misc", "norm_conv", "parallel_ops", "decay_scan", "lightning", "sink_attn", "gated_ops", "moe_sigmoid",
                            "moe_table", "moe", "glue", "dense_gemm", "stream_gemm", "tall_gemm"),
     "NilevikForCausalLM": ("api_misc", "norm_conv", "parallel_ops", "lightning", "sink_attn", "delta_rule", "gated_ops", "glue",
+                           "dense_gemm", "stream_gemm", "tall_gemm"),
+    "BanitarForCausalLM": ("api_misc", "norm_conv", "tanh_norm", "parallel_ops", "latent_attn", "sink_attn", "gated_ops", "glue",
                            "dense_gemm", "stream_gemm", "tall_gemm"),
 }
 
