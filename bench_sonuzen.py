@@ -107,6 +107,14 @@ class SonuzenRunner:
             context_lens_tensor=context_lens, block_tables=block_tables, use_cuda_graph=q == 1, max_query_len=q, max_decode_query_len=1,
             query_start_loc=qsl, seq_start_loc=None)
 
+    def _state_inputs(self, B):
+        """What a model with a state per sequence is told about its slots (nothing for one whose past is all in its pages)."""
+        if not hasattr(self.model, "get_seqlen_agnostic_capture_inputs"):
+            return {}
+        cache, idx = self.model.get_seqlen_agnostic_capture_inputs(B)
+        idx.copy_(torch.arange(B, dtype=torch.int32, device=self.dev))
+        return {"seqlen_agnostic_capture_inputs": (cache, idx)}
+
     def decode(self, B, ctx, steps, warmup):
         from vllm_hymeta import hip_ops
         dev = self.dev
@@ -121,11 +129,10 @@ class SonuzenRunner:
         slot_mapping = (torch.gather(bt.long(), 1, (positions // BLOCK).unsqueeze(1)).squeeze(1) * BLOCK + positions % BLOCK).contiguous()
         ids = torch.randint(0, self.model.config.vocab_size, (B,), generator=g).to(dev)
         md = self._metadata(B, 1, ctx, bt, slot_mapping, seq_lens, context_lens, ctx + steps + warmup + 8)
-        cache, idx = self.model.get_seqlen_agnostic_capture_inputs(B)
-        idx.copy_(torch.arange(B, dtype=torch.int32, device=dev))
+        state = self._state_inputs(B)
 
         def step():
-            h = self.model(ids, positions, attn_metadata=md, seqlen_agnostic_capture_inputs=(cache, idx))
+            h = self.model(ids, positions, attn_metadata=md, **state)
             hip_ops.argmax_rows(self.model.compute_logits(h), out=ids)
 
         for _ in range(2):
@@ -165,11 +172,10 @@ class SonuzenRunner:
                             torch.zeros(1, dtype=torch.int32, device=dev), L)
         ids = torch.randint(0, self.model.config.vocab_size, (L,), device=dev)
         pos = torch.arange(L, dtype=torch.int64, device=dev)
-        cache, idx = self.model.get_seqlen_agnostic_capture_inputs(1)
-        idx.zero_()
+        state = self._state_inputs(1)
 
         def run():
-            h = self.model(ids, pos, attn_metadata=md, seqlen_agnostic_capture_inputs=(cache, idx))
+            h = self.model(ids, pos, attn_metadata=md, **state)
             return hip_ops.argmax_rows(self.model.compute_logits(h[-1:]))
 
         run()

@@ -1366,11 +1366,12 @@ typedef struct hymeta_latent_kv_prep_args {
 int hymeta_latent_kv_prep(const hymeta_latent_kv_prep_args* args, hymeta_stream_t stream);
 
 /* The queries of a latent attention against the cached rows: out[t, h] = (q_abs[h, t] (kv_rank values: the unrotated
- * query part carried through the keys' up projection), rotated q[t, h, dim:] (rot_dim values, pairs as above)). */
+ * query part carried through the keys' up projection), rotated q[t, h, dim:] (rot_dim values, pairs as above)).  q_abs NULL:
+ * the first kv_rank values of out are in place already (the product wrote them there). */
 typedef struct hymeta_latent_q_assemble_args {
   uint32_t struct_size;
   const void* q;               /* act_dtype [num_tokens, num_heads, dim + rot_dim], row stride q_stride_t */
-  const void* q_abs;           /* act_dtype [num_heads, num_tokens, kv_rank] contiguous */
+  const void* q_abs;           /* act_dtype [num_heads, num_tokens, kv_rank] contiguous, or NULL */
   void* out;                   /* act_dtype [num_tokens, num_heads, kv_rank + rot_dim] contiguous */
   const double* rot_freqs;
   const int32_t* query_start_loc;
@@ -1765,6 +1766,9 @@ typedef struct hymeta_tanh_stream_args {
   int64_t x_stride_t, y_stride_t, base_stride_t;
 } hymeta_tanh_stream_args;
 int hymeta_tanh_stream(const hymeta_tanh_stream_args* args, hymeta_stream_t stream);
+/* hymeta_tanh_stream with y = a bf16 linear's result taken from its partial sums (args->y is ignored; num_tokens == M,
+ * width == N; act_dtype bf16; every pointer and stride in whole fours). */
+int hymeta_tanh_stream_partials(const hymeta_tanh_stream_args* args, const hymeta_gemm_partials* partials, hymeta_stream_t stream);
 
 #ifdef __cplusplus
 }

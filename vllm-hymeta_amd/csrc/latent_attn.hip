@@ -94,6 +94,31 @@ __global__ __launch_bounds__(256) void latent_kv_prep_kernel(hymeta_latent_kv_pr
   }
 }
 
+// The rotated part alone (the absorbed part is in place): grid = tokens, a (head, pair) per thread and round.
+template <typename A>
+__global__ __launch_bounds__(256) void latent_q_rotate_kernel(hymeta_latent_q_assemble_args a) {
+  typedef typename A::elem elem;
+  __shared__ float s_cos[kMaxRotPairs], s_sin[kMaxRotPairs];
+  const int t = blockIdx.x;
+  const int s = seq_of_row(a.query_start_loc, a.num_seqs, t);
+  const int pos = a.seq_lens[s] - (a.query_start_loc[s + 1] - t);
+  const int pairs = a.rot_dim / 2, C = a.kv_rank;
+  const elem* q = static_cast<const elem*>(a.q) + static_cast<int64_t>(t) * a.q_stride_t + a.dim;
+  elem* out = static_cast<elem*>(a.out) + static_cast<int64_t>(t) * a.num_heads * (C + a.rot_dim) + C;
+  fill_rotation(s_cos, s_sin, a.rot_freqs, pairs, a.rot_dims / 2, pos < 0 ? 0 : pos, a.rot_mag);
+  __syncthreads();
+  for (int idx = threadIdx.x; idx < a.num_heads * pairs; idx += 256) {
+    const int h = idx / pairs, i = idx % pairs;
+    const elem* qr = q + static_cast<int64_t>(h) * (a.dim + a.rot_dim);
+    elem* o = out + static_cast<int64_t>(h) * (C + a.rot_dim);
+    int p, r;
+    pair_at(i, a.rot_dims / 2, a.rot_half != 0, &p, &r);
+    const float u = A::ld(qr + p), v = A::ld(qr + r);
+    A::st(o + p, u * s_cos[i] - v * s_sin[i]);
+    A::st(o + r, v * s_cos[i] + u * s_sin[i]);
+  }
+}
+
 template <typename A>
 __global__ __launch_bounds__(256) void latent_q_assemble_kernel(hymeta_latent_q_assemble_args a) {
   typedef typename A::elem elem;
@@ -162,9 +187,15 @@ extern "C" int hymeta_latent_q_assemble(const hymeta_latent_q_assemble_args* arg
   if (!act_dtype_ok(a.act_dtype)) return HYMETA_ERR_UNSUPPORTED;
   if (a.rot_dim / 2 > kMaxRotPairs) return HYMETA_ERR_UNSUPPORTED;
   if (a.num_tokens == 0 || a.num_seqs == 0) return HYMETA_OK;
-  if (!a.q || !a.q_abs || !a.out || !a.query_start_loc || !a.seq_lens || (a.rot_dims > 0 && !a.rot_freqs)) return HYMETA_ERR_INVALID_ARG;
+  if (!a.q || !a.out || !a.query_start_loc || !a.seq_lens || (a.rot_dims > 0 && !a.rot_freqs)) return HYMETA_ERR_INVALID_ARG;
   if (a.q_stride_t < static_cast<int64_t>(a.num_heads) * (a.dim + a.rot_dim)) return HYMETA_ERR_INVALID_ARG;
   hipStream_t st = begin_launches(stream);
+  if (a.q_abs == nullptr) {
+    if (a.rot_dim == 0) return HYMETA_OK;
+    if (a.act_dtype == HYMETA_BF16) hipLaunchKernelGGL(latent_q_rotate_kernel<ActBf16>, dim3(a.num_tokens), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL(latent_q_rotate_kernel<ActF32>, dim3(a.num_tokens), dim3(256), 0, st, a);
+    return launch_status();
+  }
   if (a.act_dtype == HYMETA_BF16) hipLaunchKernelGGL(latent_q_assemble_kernel<ActBf16>, dim3(a.num_tokens), dim3(256), 0, st, a);
   else hipLaunchKernelGGL(latent_q_assemble_kernel<ActF32>, dim3(a.num_tokens), dim3(256), 0, st, a);
   return launch_status();

@@ -2,6 +2,7 @@
 // row): the sum of a sublayer's normed output onto the fp32 stream and the next sublayer's normed input in one elementwise
 // launch; a pass of a repeated run of layers starts the stream anew from sums of products.
 #include "act_types.h"
+#include "partial_sums.h"
 
 namespace hymeta {
 
@@ -34,8 +35,10 @@ struct Columns<A, 1> {
 
 // grid = (runs of 256 N columns, strips of R rows): a thread takes N consecutive columns through R rows, the columns'
 // constants in registers, the rows' loads in flight together.
-template <typename A, int N, int R>
-__global__ __launch_bounds__(256) void tanh_stream_kernel(hymeta_tanh_stream_args a) {
+// Partials: y is the sum of a K-sliced linear's slabs, added as it is read (N == 4, R == 1).
+template <typename A, int N, int R, bool Partials>
+__global__ __launch_bounds__(256) void tanh_stream_kernel(hymeta_tanh_stream_args a, hymeta_gemm_partials p) {
+  static_assert(!Partials || (N == 4 && R == 1), "slabs are read in fours, a row at a time");
   typedef typename A::elem elem;
   typedef Columns<ActF32, N> F;
   typedef Columns<A, N> E;
@@ -52,7 +55,13 @@ __global__ __launch_bounds__(256) void tanh_stream_kernel(hymeta_tanh_stream_arg
     const int64_t t = t0 + r;
     if (a.base) F::ld(a.base + t * a.base_stride_t + c, v[r]);
     else F::ld(a.x + t * a.x_stride_t + c, v[r]);
-    if (y) E::ld(y + t * a.y_stride_t + c, yv[r]);
+    if constexpr (Partials) {
+      const f32x4 s = partial_row4<false>(p, t, c);
+#pragma unroll
+      for (int e = 0; e < N; ++e) yv[r][e] = s[e];
+    } else if (y) {
+      E::ld(y + t * a.y_stride_t + c, yv[r]);
+    }
   }
   if (a.base) {
     float add[N];
@@ -70,7 +79,8 @@ __global__ __launch_bounds__(256) void tanh_stream_kernel(hymeta_tanh_stream_arg
       for (int e = 0; e < N; ++e) v[r][e] += b2[e] + add[e];
     }
   }
-  if (y) {
+  const bool adds = Partials || y != nullptr;
+  if (adds) {
     float w[N], b[N];
     F::ld(a.y_weight + c, w);
     F::ld(a.y_bias + c, b);
@@ -81,7 +91,7 @@ __global__ __launch_bounds__(256) void tanh_stream_kernel(hymeta_tanh_stream_arg
       for (int e = 0; e < N; ++e) v[r][e] += fmaf(squash<A>(a.y_alpha * yv[r][e]), w[e], b[e]);
     }
   }
-  if (a.base || y) {
+  if (a.base || adds) {
 #pragma unroll
     for (int r = 0; r < R; ++r)
       if (r < rows) F::st(a.x + (t0 + r) * a.x_stride_t + c, v[r]);
@@ -108,8 +118,16 @@ template <typename A, int N>
 void launch_tanh_stream(const hymeta_tanh_stream_args& a, hipStream_t st) {
   const int runs = (a.width + 256 * N - 1) / (256 * N);
   // few rows: a row per workgroup, so that there are workgroups enough
-  if (a.num_tokens >= 1024) hipLaunchKernelGGL((tanh_stream_kernel<A, N, kStripRows>), dim3(runs, (a.num_tokens + kStripRows - 1) / kStripRows), dim3(256), 0, st, a);
-  else hipLaunchKernelGGL((tanh_stream_kernel<A, N, 1>), dim3(runs, a.num_tokens), dim3(256), 0, st, a);
+  if (a.num_tokens >= 1024) hipLaunchKernelGGL((tanh_stream_kernel<A, N, kStripRows, false>), dim3(runs, (a.num_tokens + kStripRows - 1) / kStripRows), dim3(256), 0, st, a, hymeta_gemm_partials{});
+  else hipLaunchKernelGGL((tanh_stream_kernel<A, N, 1, false>), dim3(runs, a.num_tokens), dim3(256), 0, st, a, hymeta_gemm_partials{});
+}
+
+inline bool whole_fours(const void* p, int64_t stride, int bytes) { return p == nullptr || (reinterpret_cast<uintptr_t>(p) % (4 * bytes) == 0 && stride % 4 == 0); }
+// Everything but y in whole fours of columns.
+inline bool stream_in_fours(const hymeta_tanh_stream_args& a, int eb) {
+  return a.width % 4 == 0 && whole_fours(a.x, a.x_stride_t, 4) && whole_fours(a.base, a.base_stride_t, 4) && whole_fours(a.base2, a.base_stride_t, 4) &&
+         whole_fours(a.add, 0, 4) && whole_fours(a.y_weight, 0, 4) && whole_fours(a.y_bias, 0, 4) && whole_fours(a.h_weight, 0, 4) &&
+         whole_fours(a.h_bias, 0, 4) && whole_fours(a.h_out, 0, eb);
 }
 
 }  // namespace
@@ -131,10 +149,7 @@ extern "C" int hymeta_tanh_stream(const hymeta_tanh_stream_args* args, hymeta_st
   if ((a.num_tokens + kStripRows - 1) / kStripRows > 65535) return HYMETA_ERR_UNSUPPORTED;
   hipStream_t st = begin_launches(stream);
   const int eb = a.act_dtype == HYMETA_BF16 ? 2 : 4;
-  auto fours = [](const void* p, int64_t stride, int bytes) { return p == nullptr || (reinterpret_cast<uintptr_t>(p) % (4 * bytes) == 0 && stride % 4 == 0); };
-  const bool vec = a.width % 4 == 0 && fours(a.x, a.x_stride_t, 4) && fours(a.y, a.y_stride_t, eb) && fours(a.base, a.base_stride_t, 4) &&
-                   fours(a.base2, a.base_stride_t, 4) && fours(a.add, 0, 4) && fours(a.y_weight, 0, 4) && fours(a.y_bias, 0, 4) &&
-                   fours(a.h_weight, 0, 4) && fours(a.h_bias, 0, 4) && fours(a.h_out, 0, eb);
+  const bool vec = stream_in_fours(a, eb) && whole_fours(a.y, a.y_stride_t, eb);
   if (a.act_dtype == HYMETA_BF16) {
     if (vec) launch_tanh_stream<ActBf16, 4>(a, st);
     else launch_tanh_stream<ActBf16, 1>(a, st);
@@ -142,5 +157,19 @@ extern "C" int hymeta_tanh_stream(const hymeta_tanh_stream_args* args, hymeta_st
     if (vec) launch_tanh_stream<ActF32, 4>(a, st);
     else launch_tanh_stream<ActF32, 1>(a, st);
   }
+  return launch_status();
+}
+
+extern "C" int hymeta_tanh_stream_partials(const hymeta_tanh_stream_args* args, const hymeta_gemm_partials* partials, hymeta_stream_t stream) {
+  if (!args_ok(args) || !args_ok(partials)) return HYMETA_ERR_INVALID_ARG;
+  const hymeta_tanh_stream_args& a = *args;
+  const hymeta_gemm_partials& p = *partials;
+  if (a.num_tokens < 0 || a.width <= 0 || p.splits <= 0 || p.is_int32 || !p.slabs || p.M != a.num_tokens || p.N != a.width) return HYMETA_ERR_INVALID_ARG;
+  if (a.act_dtype != HYMETA_BF16) return HYMETA_ERR_UNSUPPORTED;
+  if (a.num_tokens == 0) return HYMETA_OK;
+  if (!a.x || a.x_stride_t < a.width || !a.y_weight || !a.y_bias || a.base || a.base2 || a.add || (a.h_weight && !a.h_bias)) return HYMETA_ERR_INVALID_ARG;
+  if (!stream_in_fours(a, 2) || reinterpret_cast<uintptr_t>(p.slabs) % 16 != 0 || !whole_fours(p.bias, 0, 2) || a.num_tokens > 65535) return HYMETA_ERR_UNSUPPORTED;
+  hipStream_t st = begin_launches(stream);
+  hipLaunchKernelGGL((tanh_stream_kernel<ActBf16, 4, 1, true>), dim3((a.width + 1023) / 1024, a.num_tokens), dim3(256), 0, st, a, p);
   return launch_status();
 }

@@ -707,6 +707,7 @@ _SIGNATURES = {
     "hymeta_stream_add_norm": (C.c_int, [C.POINTER(StreamAddNormArgs), _ptr]),
     "hymeta_rotary_cache": (C.c_int, [C.POINTER(RotaryCacheArgs), _ptr]),
     "hymeta_tanh_stream": (C.c_int, [C.POINTER(TanhStreamArgs), _ptr]),
+    "hymeta_tanh_stream_partials": (C.c_int, [C.POINTER(TanhStreamArgs), C.POINTER(GemmPartials), _ptr]),
     "hymeta_causal_conv": (C.c_int, [C.POINTER(CausalConvArgs), _ptr]),
     "hymeta_decay_scan_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32]),
     "hymeta_decay_scan": (C.c_int, [C.POINTER(DecayScanArgs), _ptr]),

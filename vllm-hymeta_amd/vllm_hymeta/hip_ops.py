@@ -1892,6 +1892,26 @@ def latent_kv_prep_(proj: torch.Tensor, q_col: int, q_rank: int, kv_col: int, kv
     _C.check(_C.load().hymeta_latent_kv_prep(C.byref(a), _stream(proj)), "hymeta_latent_kv_prep")
 
 
+def latent_q_rotate_(out: torch.Tensor, q: torch.Tensor, dim: int, rot_dim: int, rot_dims: int, rot_freqs: torch.Tensor, rot_mag: float,
+                     query_start_loc: torch.Tensor, seq_lens: torch.Tensor, rot_half: bool = False) -> None:
+    """``out [T, H, C + rot_dim]`` whose first ``C`` columns the absorbing product wrote: the rest becomes the rotated part of
+    ``q [T, H, dim + rot_dim]``."""
+    _dev(out, q, rot_freqs, query_start_loc, seq_lens)
+    _require(q.dim() == 3 and q.stride(2) == 1 and q.stride(1) == dim + rot_dim and q.shape[2] == dim + rot_dim, "q must be [T, H, dim + rot_dim]")
+    T, H, _ = q.shape
+    _require(out.dim() == 3 and out.is_contiguous() and out.shape[:2] == (T, H) and out.shape[2] > rot_dim and out.dtype == q.dtype,
+             "out must be contiguous [T, H, C + rot_dim] of q's type")
+    _require(rot_freqs.dtype == torch.float64 and rot_freqs.is_contiguous() and rot_freqs.numel() * 2 >= rot_dims, "rot_freqs must be float64 [rot_dims / 2]")
+    S = query_start_loc.numel() - 1
+    _i32vec(query_start_loc, S + 1, "query_start_loc")
+    _i32vec(seq_lens, S, "seq_lens")
+    a = _C.LatentQAssembleArgs()
+    a.q, a.out, a.rot_freqs, a.query_start_loc, a.seq_lens = _p(q), _p(out), _p(rot_freqs), _p(query_start_loc), _p(seq_lens)
+    a.num_tokens, a.num_seqs, a.num_heads, a.dim, a.rot_dim, a.rot_dims, a.kv_rank, a.act_dtype = T, S, H, dim, rot_dim, rot_dims, out.shape[2] - rot_dim, _act(q)
+    a.rot_mag, a.q_stride_t, a.rot_half = rot_mag, q.stride(0), int(rot_half)
+    _C.check(_C.load().hymeta_latent_q_assemble(C.byref(a), _stream(q)), "hymeta_latent_q_assemble")
+
+
 def latent_q_assemble(q: torch.Tensor, q_abs: torch.Tensor, dim: int, rot_dim: int, rot_dims: int, rot_freqs: torch.Tensor,
                       rot_mag: float, query_start_loc: torch.Tensor, seq_lens: torch.Tensor, rot_half: bool = False) -> torch.Tensor:
     """``q [T, H, dim + rot_dim]`` and ``q_abs [H, T, C]`` -> ``[T, H, C + rot_dim]``: the absorbed part followed by the
@@ -2494,26 +2514,29 @@ class SquashNorm(NamedTuple):
     bias: torch.Tensor            # fp32 [W]
 
 
-def tanh_stream_(x: torch.Tensor, y: Optional[torch.Tensor] = None, y_norm: Optional[SquashNorm] = None, base: Optional[torch.Tensor] = None,
+def tanh_stream_(x: torch.Tensor, y=None, y_norm: Optional[SquashNorm] = None, base: Optional[torch.Tensor] = None,
                  base2: Optional[torch.Tensor] = None, add: Optional[torch.Tensor] = None, read: Optional[SquashNorm] = None,
                  out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
     """On the fp32 stream ``x [T, W]``, in place, one launch: ``x = base (+ base2) (+ add)`` with ``base`` (fp32 ``[T, W]``), then
-    ``x += y_norm(y)`` with ``y``.  ``out_dtype``: returns ``read(x)`` (without ``read``: ``x``) in that type."""
-    _dev(x, y, base, base2, add, *(t for n in (y_norm, read) if n is not None for t in (n.weight, n.bias)))
+    ``x += y_norm(y)`` with ``y`` (a tensor, or the ``PartialSums`` of a K-sliced linear: the slices are added as they are read).  ``out_dtype``: returns ``read(x)`` (without ``read``: ``x``) in that type."""
+    partials = y if isinstance(y, PartialSums) else None
+    _dev(x, None if partials else y, base, base2, add, *(t for n in (y_norm, read) if n is not None for t in (n.weight, n.bias)))
     _require(x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1, "x must be row-contiguous fp32 [T, W]")
     _require((y is None) == (y_norm is None), "y comes with its norm")
     _require(y is not None or base is not None or out_dtype is not None, "nothing to do")
     T, W = x.shape
     a = _C.TanhStreamArgs()
     a.x, a.num_tokens, a.width, a.x_stride_t = _p(x), T, W, x.stride(0)
-    act = y.dtype if y is not None else (out_dtype or torch.float32)
+    act = torch.bfloat16 if partials else y.dtype if y is not None else (out_dtype or torch.float32)
     _require(out_dtype is None or out_dtype == act, "the sublayers' activations have one type")
     _require(act in _DT, "activations must be bf16 or fp32")
     a.act_dtype = _DT[act]
     if y is not None:
-        _require(y.shape == (T, W) and y.stride(1) == 1, "y must be row-contiguous [T, W]")
+        _require(tuple(y.shape) == (T, W) and (partials is not None or y.stride(1) == 1), "y must be row-contiguous [T, W]")
         _f32vec(y_norm.weight, W, "y_norm.weight"), _f32vec(y_norm.bias, W, "y_norm.bias")
-        a.y, a.y_stride_t, a.y_alpha, a.y_weight, a.y_bias = _p(y), y.stride(0), float(y_norm.alpha), _p(y_norm.weight), _p(y_norm.bias)
+        a.y_alpha, a.y_weight, a.y_bias = float(y_norm.alpha), _p(y_norm.weight), _p(y_norm.bias)
+        if partials is None:
+            a.y, a.y_stride_t = _p(y), y.stride(0)
     if base is not None:
         for b in (base, base2):
             _require(b is None or (b.shape == (T, W) and b.dtype == torch.float32 and b.stride(1) == 1 and b.stride(0) == base.stride(0)),
@@ -2529,5 +2552,10 @@ def tanh_stream_(x: torch.Tensor, y: Optional[torch.Tensor] = None, y_norm: Opti
         if read is not None:
             _f32vec(read.weight, W, "read.weight"), _f32vec(read.bias, W, "read.bias")
             a.h_weight, a.h_bias, a.h_alpha = _p(read.weight), _p(read.bias), float(read.alpha)
+    if partials is not None:
+        _require(base is None, "partial sums are added to the stream")
+        partials.check_live()
+        _C.check(_C.load().hymeta_tanh_stream_partials(C.byref(a), C.byref(partials.desc), _stream(x)), "hymeta_tanh_stream_partials")
+        return h
     _C.check(_C.load().hymeta_tanh_stream(C.byref(a), _stream(x)), "hymeta_tanh_stream")
     return h

@@ -75,11 +75,12 @@ class SiluGluMLP(torch.nn.Module):
         super().__init__()
         self.gate_up_proj, self.down_proj = gate_up_proj, down_proj
 
-    def forward(self, h: torch.Tensor) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, defer: bool = False):
+        """``defer``: the down projection may leave its slices' sum to the caller (``HymetaLinear.forward``)."""
         gu = self.gate_up_proj
         if gu.bias is None and hip_ops.gemm_silu_mul_supported(h, gu.weight):      # decode-sized bf16 batches: in the GEMM's epilogue
-            return self.down_proj(hip_ops.gemm_silu_mul(h, gu.weight))
-        return self.down_proj(hip_ops.silu_mul(gu(h)))
+            return self.down_proj(hip_ops.gemm_silu_mul(h, gu.weight), defer=defer)
+        return self.down_proj(hip_ops.silu_mul(gu(h)), defer=defer)
 
 
 class GeluGluMLP(torch.nn.Module):

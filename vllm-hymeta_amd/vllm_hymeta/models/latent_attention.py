@@ -82,7 +82,8 @@ class LatentAttentionMixer(torch.nn.Module):
         self.rot_half, self.q_cols = bool(rot_half), q_rank or num_heads * (dim + rot_dim)        # columns ahead of the key/value latent
         self._attn = (attn,)          # owned (and registered as a module) by the model, one per layer that runs these weights
 
-    def forward(self, h: torch.Tensor, layout, attn: Optional[PagedLatentAttention] = None) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, layout, attn: Optional[PagedLatentAttention] = None, defer: bool = False):
+        """``defer``: the output projection may leave its slices' sum to the caller (``HymetaLinear.forward``)."""
         attn = attn or self._attn[0]
         H, D, R, Dv, C, Q, cols = self.H, self.D, self.R, self.Dv, self.C, self.Q, self.q_cols
         T = h.shape[0]
@@ -90,11 +91,13 @@ class LatentAttentionMixer(torch.nn.Module):
         hip_ops.latent_kv_prep_(proj, 0, Q, cols, C, R, self.rot_dims, self.q_norm_weight, self.kv_norm_weight, self.eps, self.rot_freqs,
                                 self.rot_mag, attn.cache(), layout.slot_mapping, layout.query_start_loc, layout.seq_lens, self.rot_half)
         q = (proj[:, :cols] if self.uq_proj is None else self.uq_proj(proj[:, :Q])).view(T, H, D + R)
-        q_abs = torch.bmm(q[:, :, :D].transpose(0, 1), self.uk)                       # [H, T, C]
-        q_full = hip_ops.latent_q_assemble(q, q_abs, D, R, self.rot_dims, self.rot_freqs, self.rot_mag, layout.query_start_loc,
-                                           layout.seq_lens, self.rot_half)
+        # the two batched products (a head each) write where their readers want the heads: a token's side by side
+        q_full = torch.empty(T, H, C + R, dtype=h.dtype, device=h.device)
+        torch.bmm(q[:, :, :D].transpose(0, 1), self.uk, out=q_full[:, :, :C].transpose(0, 1))
+        hip_ops.latent_q_rotate_(q_full, q, D, R, self.rot_dims, self.rot_freqs, self.rot_mag, layout.query_start_loc, layout.seq_lens, self.rot_half)
         o_lat = attn(q_full, layout)                                                  # [T, H, C]
-        o = torch.bmm(o_lat.transpose(0, 1), self.uv).transpose(0, 1).reshape(T, H * Dv)
+        o = torch.empty(T, H * Dv, dtype=h.dtype, device=h.device)
+        torch.bmm(o_lat.transpose(0, 1), self.uv, out=o.view(T, H, Dv).transpose(0, 1))
         if self.gate:
             o = hip_ops.sigmoid_gate_mul(o, proj[:, cols + C + R:cols + C + R + H * Dv])
-        return self.o_proj(o)
+        return self.o_proj(o, defer=defer)

@@ -71,7 +71,8 @@ class WindowAttentionMixer(torch.nn.Module):
         self.register_buffer("rot_freqs", None if rot_freqs is None else rot_freqs.to(torch.float64).contiguous())
         self._attn = (attn,)          # owned (and registered as a module) by the model, one per layer that runs these weights
 
-    def forward(self, h: torch.Tensor, layout, attn: Optional[PagedWindowAttention] = None) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, layout, attn: Optional[PagedWindowAttention] = None, defer: bool = False):
+        """``defer``: the output projection may leave its slices' sum to the caller (``HymetaLinear.forward``)."""
         attn = attn or self._attn[0]
         H, G, D, Dv = attn.num_heads, attn.num_kv_heads, attn.head_size, attn.v_size
         proj = self.in_proj(h)
@@ -80,4 +81,4 @@ class WindowAttentionMixer(torch.nn.Module):
                               interleaved=self.interleaved, rot_mag=self.rot_mag, unit_eps=self.unit_eps)
         gate = proj[:, (H + G) * D + G * Dv:(H + G) * D + G * Dv + H] if self.gated else None
         o = attn(proj[:, :H * D].view(-1, H, D), layout, gate)
-        return self.o_proj(o.view(-1, H * Dv))
+        return self.o_proj(o.view(-1, H * Dv), defer=defer)

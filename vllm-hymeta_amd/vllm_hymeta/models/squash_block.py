@@ -43,16 +43,18 @@ class TanhNorm(torch.nn.Module):
         return hip_ops.tanh_stream_(x, read=self.constants, out_dtype=out_dtype)
 
 
-def add_and_read(x: torch.Tensor, y: torch.Tensor, out_norm: TanhNorm, read: Optional[TanhNorm]) -> torch.Tensor:
-    """``x += out_norm(y)``; returns what the next sublayer reads, in y's type: ``read(x)``, or (None) the stream itself."""
-    if read is None and y.dtype == torch.float32:
+def add_and_read(x: torch.Tensor, y, out_norm: TanhNorm, read: Optional[TanhNorm], act_dtype: torch.dtype) -> torch.Tensor:
+    """``x += out_norm(y)``, ``y`` a sublayer's output or the partial sums of its last projection; returns what the next sublayer
+    reads: ``read(x)``, or (None) the stream itself."""
+    if read is None and act_dtype == torch.float32:
         hip_ops.tanh_stream_(x, y, out_norm.constants)
         return x
-    return hip_ops.tanh_stream_(x, y, out_norm.constants, read=None if read is None else read.constants, out_dtype=y.dtype)
+    return hip_ops.tanh_stream_(x, y, out_norm.constants, read=None if read is None else read.constants, out_dtype=act_dtype)
 
 
 class SquashBlock(torch.nn.Module):
-    """One decoder layer.  ``mixer(h, layout, state)`` and ``mlp(h)`` take and return activations; ``mlp`` may be absent."""
+    """One decoder layer.  ``mixer(h, layout, state, defer=True)`` and ``mlp(h, defer=True)`` take activations and return them,
+    or the partial sums of their last projection; ``mlp`` may be absent."""
 
     def __init__(self, mixer_in: TanhNorm, mixer: torch.nn.Module, mixer_out: TanhNorm, mlp_in: Optional[TanhNorm] = None,
                  mlp: Optional[torch.nn.Module] = None, mlp_out: Optional[TanhNorm] = None):
@@ -62,10 +64,12 @@ class SquashBlock(torch.nn.Module):
 
     def forward(self, x: torch.Tensor, h: torch.Tensor, layout: StepLayout, mixer_state, read: Optional[TanhNorm]) -> torch.Tensor:
         """``h``: ``mixer_in`` of the stream.  Returns ``read`` of the stream after the layer (None: its copy)."""
-        y = self.mixer(h, layout, mixer_state)
+        act = h.dtype
+        y = self.mixer(h, layout, mixer_state, defer=True)
         if self.mlp is None:
-            return add_and_read(x, y, self.mixer_out, read)
-        return add_and_read(x, self.mlp(add_and_read(x, y, self.mixer_out, self.mlp_in)), self.mlp_out, read)
+            return add_and_read(x, y, self.mixer_out, read, act)
+        h = add_and_read(x, y, self.mixer_out, self.mlp_in, act)
+        return add_and_read(x, self.mlp(h, defer=True), self.mlp_out, read, act)
 
 
 class PassEntry(torch.nn.Module):
