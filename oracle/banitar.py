@@ -54,12 +54,12 @@ def rotate_ref(x: torch.Tensor, dims: int, freqs: List[float], mag: float, half_
     """``x [T, heads, D]``, row t at position t: the first ``dims`` dimensions turn in pairs, ``(i, i + dims / 2)`` with
     ``half_split``, else ``(2 i, 2 i + 1)``."""
     out = x.clone()
-    for t in range(x.shape[0]):
-        for i in range(dims // 2):
-            p, r = (i, i + dims // 2) if half_split else (2 * i, 2 * i + 1)
-            c, s = math.cos(t * freqs[i]) * mag, math.sin(t * freqs[i]) * mag
-            u, v = x[t, :, p], x[t, :, r]
-            out[t, :, p], out[t, :, r] = u * c - v * s, v * c + u * s
+    t = torch.arange(x.shape[0], dtype=torch.float64)
+    for i in range(dims // 2):
+        p, r = (i, i + dims // 2) if half_split else (2 * i, 2 * i + 1)
+        c, s = ((f(t * freqs[i]) * mag).to(x.dtype)[:, None] for f in (torch.cos, torch.sin))
+        u, v = x[:, :, p], x[:, :, r]
+        out[:, :, p], out[:, :, r] = u * c - v * s, v * c + u * s
     return out
 
 
